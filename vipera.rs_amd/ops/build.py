@@ -3,7 +3,7 @@
 Each module is one shared library built from a few source files with ``hipcc`` (kernels) or
 ``g++`` (host code).  A library is named after a hash of its sources and flags, so a library
 that is present is always the one its sources describe.  A module is compiled the first time
-something asks for it; while a compile runs, a line is printed every few seconds.  Libraries go
+something asks for it; a line is printed when a compile starts and when it has ended.  Libraries go
 to ``csrc/_build`` inside the package, or to a per-user folder under the temporary directory when
 the package folder cannot be written.
 """
@@ -120,20 +120,8 @@ def compile_module(name: str, verbose: bool = True) -> str:
     started = time.time()
     if verbose:
         print(f"[vipera build] compiling {name} ({', '.join(sources)})", file=sys.stderr, flush=True)
-    process = subprocess.Popen(command, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
-    output: List[str] = []
-    reader = threading.Thread(target=lambda: output.append(process.stdout.read()), daemon=True)
-    reader.start()
-    while True:
-        try:
-            process.wait(timeout=10)
-            break
-        except subprocess.TimeoutExpired:
-            if verbose:
-                print(f"[vipera build] still compiling {name} ... {time.time() - started:.0f} s",
-                      file=sys.stderr, flush=True)
-    reader.join()
-    text = "\n".join(line for line in "".join(output).splitlines() if "not a recognized feature" not in line)
+    process = subprocess.run(command, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
+    text = "\n".join(line for line in process.stdout.splitlines() if "not a recognized feature" not in line)
     if process.returncode != 0:
         if os.path.exists(tmp):
             os.remove(tmp)
