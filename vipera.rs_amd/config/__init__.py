@@ -3,6 +3,7 @@ from .gilidra import GilidraConfig
 from .lurirax import LuriraxConfig
 from .muzasun import MuzasunConfig
 from .qwen2 import Qwen2Config
+from .zeladra import ZeladraConfig
 from .zulesun import ZulesunConfig
 from .registry import (
     architecture_names,
@@ -16,6 +17,7 @@ from .registry import (
 
 __all__ = [
     "KeyReader", "LayerSpec", "ModelConfig", "PartSpec", "ScheduleEntry", "read_config_json",
-    "GilidraConfig", "LuriraxConfig", "MuzasunConfig", "Qwen2Config", "ZulesunConfig", "architecture_names", "architecture_of", "config_from_dict", "load_config",
+    "GilidraConfig", "LuriraxConfig", "MuzasunConfig", "Qwen2Config", "ZeladraConfig", "ZulesunConfig",
+    "architecture_names", "architecture_of", "config_from_dict", "load_config",
     "lookup_architecture", "register_architecture", "unregister_architecture",
 ]

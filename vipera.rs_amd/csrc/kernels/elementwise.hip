@@ -48,31 +48,38 @@ extern "C" int vk_fetch_words(const void* pinned_host, void* out, long long coun
 template <typename TW>
 __global__ void embed_gather_kernel(const TW* __restrict__ table, const int* __restrict__ tokens,
                                     const int* __restrict__ source, const int* __restrict__ sampled,
-                                    float* __restrict__ out, int width, int vocab) {
+                                    float* __restrict__ out, int width, int vocab, float scale) {
   const int t = blockIdx.x;
   int token = tokens[t];
   if (source != nullptr && source[t] >= 0) token = sampled[source[t]];
   if (token < 0 || token >= vocab) token = 0;
   const TW* row = table + (size_t)token * width;
   float* dst = out + (size_t)t * width;
-  for (int i = threadIdx.x; i < width; i += blockDim.x) dst[i] = to_float<TW>(row[i]);
+  for (int i = threadIdx.x; i < width; i += blockDim.x) dst[i] = to_float<TW>(row[i]) * scale;
 }
 
-extern "C" int vk_embed_gather(const void* table, int table_dtype, const int* tokens, const int* source,
-                               const int* sampled, float* out, int num_tokens, int width, int vocab, void* stream) {
+// `scale` multiplies the rows (a model whose embedding is scaled).
+extern "C" int vk_embed_gather_scaled(const void* table, int table_dtype, const int* tokens, const int* source,
+                                      const int* sampled, float* out, int num_tokens, int width, int vocab, float scale,
+                                      void* stream) {
   if (num_tokens <= 0) return 0;
   if (width <= 0 || vocab <= 0 || (source != nullptr && sampled == nullptr)) return VK_BAD_ARGUMENT;
   hipStream_t s = (hipStream_t)stream;
   if (table_dtype == DT_F32)
     embed_gather_kernel<float><<<num_tokens, 256, 0, s>>>((const float*)table, tokens, source, sampled, out, width,
-                                                          vocab);
+                                                          vocab, scale);
   else if (table_dtype == DT_BF16)
     embed_gather_kernel<bf16_t><<<num_tokens, 256, 0, s>>>((const bf16_t*)table, tokens, source, sampled, out, width,
-                                                           vocab);
+                                                           vocab, scale);
   else
     return VK_BAD_ARGUMENT;
   VK_LAUNCH_CHECK();
   return 0;
+}
+
+extern "C" int vk_embed_gather(const void* table, int table_dtype, const int* tokens, const int* source,
+                               const int* sampled, float* out, int num_tokens, int width, int vocab, void* stream) {
+  return vk_embed_gather_scaled(table, table_dtype, tokens, source, sampled, out, num_tokens, width, vocab, 1.0f, stream);
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -157,25 +164,31 @@ extern "C" int vk_rmsnorm(const float* x, const float* weight, const int* rows, 
 // frequencies: out[t * half + i] = (sin, cos)(float(pos_t) * inv_freq[i]), the same expression in the same
 // precision as rope_kvwrite_kernel evaluates without a table (the reference keeps one table per position for
 // all layers, crates/vipera-backend-cpu/src/model.rs:4174-4181).
+// `amplitude` multiplies both (a rotation that also scales).
 __global__ void rope_angles_kernel(const int* __restrict__ positions, const float* __restrict__ inv_freq,
-                                   float2* __restrict__ out, int num_tokens, int half) {
+                                   float2* __restrict__ out, int num_tokens, int half, float amplitude) {
   const long long idx = (long long)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= (long long)num_tokens * half) return;
   const int t = (int)(idx / half), i = (int)(idx % half);
   float sn, cs;
   sincosf((float)positions[t] * inv_freq[i], &sn, &cs);
-  out[idx] = make_float2(sn, cs);
+  out[idx] = make_float2(amplitude * sn, amplitude * cs);
 }
 
-extern "C" int vk_rope_angles(const int* positions, const float* inv_freq, int half, int num_tokens, float* out,
-                              void* stream) {
+extern "C" int vk_rope_angles_scaled(const int* positions, const float* inv_freq, int half, int num_tokens, float amplitude,
+                                     float* out, void* stream) {
   if (num_tokens <= 0 || half <= 0) return 0;
   const long long total = (long long)num_tokens * half;
   if (total > 0x7fffffffLL * 256) return VK_UNSUPPORTED_SIZE;
   rope_angles_kernel<<<(unsigned)((total + 255) / 256), 256, 0, (hipStream_t)stream>>>(positions, inv_freq,
-                                                                                        (float2*)out, num_tokens, half);
+                                                                                        (float2*)out, num_tokens, half, amplitude);
   VK_LAUNCH_CHECK();
   return 0;
+}
+
+extern "C" int vk_rope_angles(const int* positions, const float* inv_freq, int half, int num_tokens, float* out,
+                              void* stream) {
+  return vk_rope_angles_scaled(positions, inv_freq, half, num_tokens, 1.0f, out, stream);
 }
 
 constexpr int ROPE_HEADS_PER_BLOCK = 4;  // one wave per head

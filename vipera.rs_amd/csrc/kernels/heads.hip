@@ -10,7 +10,7 @@ constexpr int HEAD_REGS = 4;   // a lane keeps up to four numbers of a head: hea
 // attention kernels read, every head at one padded width W.
 //   proj [T, ldp]: q (heads * maps * dim) | k (kv_heads * maps * dim) | v (kv_heads * vdim) from column 0 on
 //   rotation   the first rot_dims numbers of a q or k head in the half-split layout: pair (i, i + rot_dims / 2) turns
-//              by float(position) * inv_freq[i]; rot_dims 0: none
+//              by float(position) * inv_freq[i], sine and cosine times `amplitude`; rot_dims 0: none
 //   norm       0 none; 1 every q and k head divided by its root mean square (eps inside the root) and multiplied by a
 //              weight of `dim` numbers shared by the heads (null: no weight); norm_first: before the rotation, else
 //              behind it
@@ -27,7 +27,8 @@ template <typename TO>
 __global__ __launch_bounds__(256) void head_prepare_kernel(
     const float* __restrict__ proj, long long ldp, const float* __restrict__ q_weight, const float* __restrict__ k_weight,
     int norm, int norm_first, float eps, const int* __restrict__ positions, const float* __restrict__ inv_freq,
-    int rot_dims, int heads, int kv_heads, int maps, int dim, int vdim, int W, long long units, TO* __restrict__ qkv,
+    int rot_dims, float amplitude, int heads, int kv_heads, int maps, int dim, int vdim, int W, long long units,
+    TO* __restrict__ qkv,
     TO* __restrict__ k_cache, TO* __restrict__ v_cache, const int* __restrict__ entry_of_token,
     const int* __restrict__ block_table, int table_width, int block_size) {
   const int lane = threadIdx.x & (WAVE - 1);
@@ -98,7 +99,7 @@ __global__ __launch_bounds__(256) void head_prepare_kernel(
       if (d < rot_dims) {
         float sn, cs;
         sincosf(pos * inv_freq[d < half ? d : d - half], &sn, &cs);
-        y[i] = d < half ? y[i] * cs - partner[i] * sn : y[i] * cs + partner[i] * sn;
+        y[i] = amplitude * (d < half ? y[i] * cs - partner[i] * sn : y[i] * cs + partner[i] * sn);
       }
       ss = fmaf(y[i], y[i], ss);
     }
@@ -234,7 +235,7 @@ __global__ void row_gate_add_kernel(const float* __restrict__ y, const float* __
 
 extern "C" int vk_head_prepare(const float* proj, long long ldp, const float* q_weight, const float* k_weight, int norm,
                                int norm_first, float eps, const int* positions, const float* inv_freq, int rot_dims,
-                               int num_tokens, int heads, int kv_heads, int maps, int dim, int vdim, int W, void* qkv,
+                               float amplitude, int num_tokens, int heads, int kv_heads, int maps, int dim, int vdim, int W, void* qkv,
                                int dtype, void* k_cache, void* v_cache, const int* entry_of_token, const int* block_table,
                                int table_width, int block_size, void* stream) {
   if (num_tokens <= 0) return 0;
@@ -249,12 +250,12 @@ extern "C" int vk_head_prepare(const float* proj, long long ldp, const float* q_
   if (blocks > 0x7fffffffLL) return VK_UNSUPPORTED_SIZE;
   if (dtype == DT_F32)
     head_prepare_kernel<float><<<(unsigned)blocks, 256, 0, s>>>(proj, ldp, q_weight, k_weight, norm, norm_first, eps, positions,
-                                                                inv_freq, rot_dims, heads, kv_heads, maps, dim, vdim, W, units,
+                                                                inv_freq, rot_dims, amplitude, heads, kv_heads, maps, dim, vdim, W, units,
                                                                 (float*)qkv, (float*)k_cache, (float*)v_cache, entry_of_token,
                                                                 block_table, table_width, block_size);
   else if (dtype == DT_BF16)
     head_prepare_kernel<bf16_t><<<(unsigned)blocks, 256, 0, s>>>(proj, ldp, q_weight, k_weight, norm, norm_first, eps, positions,
-                                                                 inv_freq, rot_dims, heads, kv_heads, maps, dim, vdim, W, units,
+                                                                 inv_freq, rot_dims, amplitude, heads, kv_heads, maps, dim, vdim, W, units,
                                                                  (bf16_t*)qkv, (bf16_t*)k_cache, (bf16_t*)v_cache,
                                                                  entry_of_token, block_table, table_width, block_size);
   else

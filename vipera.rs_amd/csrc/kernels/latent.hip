@@ -11,17 +11,42 @@
 #include "group_tile.h"
 
 // ---------------------------------------------------------------------------------------------
-// One workgroup per token: c = rms_norm(x[:rank]) * weight, kr = rotate(x[rank:]) (pairs (i, i + rot_dims / 2) of
-// the first `rot_dims` dims, angle float(pos) * inv_freq[i]); the row goes to the token's page and slot.
-// x: 32-bit [T, ldx].  A token whose page id is negative writes nothing.
+// One workgroup per token, from the 32-bit row x of its down products:
+//   c = rms_norm(x[:rank]) * weight, kr = rotate(x[rank:]) (pairs (i, i + rot_dims / 2) of the first `rot_dims` dims,
+//   angle float(pos) * inv_freq[i], sine and cosine times `amplitude`); the row goes to the token's page and slot.  A token
+//   whose page id is negative writes nothing; k_cache null: no row is made.
+//   c_q = rms_norm(xq[:q_rank]) * q_weight, the queries' latent, to q_out [T, q_rank]; q_out null: not made.
 template <typename TC>
-__global__ __launch_bounds__(256) void latent_kv_write_kernel(
-    const float* __restrict__ x, long long ldx, const float* __restrict__ weight, float eps, int rank, int rot,
-    int rot_dims, const int* __restrict__ positions, const float* __restrict__ inv_freq,
+__global__ __launch_bounds__(256) void latent_prepare_kernel(
+    const float* __restrict__ x, const float* __restrict__ xq, long long ldx, const float* __restrict__ weight, float eps,
+    int rank, int rot, int rot_dims, float amplitude, const int* __restrict__ positions, const float* __restrict__ inv_freq,
     const int* __restrict__ entry_of, const int* __restrict__ table, int table_width, int block_size,
-    TC* __restrict__ k_cache, TC* __restrict__ v_cache) {
+    TC* __restrict__ k_cache, TC* __restrict__ v_cache, const float* __restrict__ q_weight, int q_rank,
+    TC* __restrict__ q_out) {
   __shared__ float scratch[16];
   const int t = blockIdx.x;
+  if (q_out) {
+    const float* src = xq + (long long)t * ldx;
+    constexpr int KEPT = 8;      // a latent of up to 2,048 numbers is read once
+    float v[KEPT], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < KEPT; ++i) {
+      const int c = threadIdx.x + 256 * i;
+      v[i] = c < q_rank ? src[c] : 0.f;
+      ss = fmaf(v[i], v[i], ss);
+    }
+    for (int c = threadIdx.x + 256 * KEPT; c < q_rank; c += 256) ss = fmaf(src[c], src[c], ss);
+    ss = block_sum(ss, scratch);
+    const float inv = 1.0f / sqrtf(ss / (float)q_rank + eps);
+    TC* dst = q_out + (long long)t * q_rank;
+#pragma unroll
+    for (int i = 0; i < KEPT; ++i) {
+      const int c = threadIdx.x + 256 * i;
+      if (c < q_rank) dst[c] = from_float<TC>(v[i] * inv * q_weight[c]);
+    }
+    for (int c = threadIdx.x + 256 * KEPT; c < q_rank; c += 256) dst[c] = from_float<TC>(src[c] * inv * q_weight[c]);
+  }
+  if (!k_cache) return;
   const float* src = x + (long long)t * ldx;
   float ss = 0.f;
   for (int c = threadIdx.x; c < rank; c += blockDim.x) ss += src[c] * src[c];
@@ -45,7 +70,7 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(
         float sn, cs;
         sincosf((float)pos * inv_freq[pair], &sn, &cs);
         const float lo = src[rank + pair], hi = src[rank + pair + half];
-        value = i < half ? lo * cs - hi * sn : hi * cs + lo * sn;
+        value = amplitude * (i < half ? lo * cs - hi * sn : hi * cs + lo * sn);
       } else {
         value = src[c];
       }
@@ -62,7 +87,7 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(
 template <typename T>
 __global__ void latent_q_rotate_kernel(const T* __restrict__ q, long long ldq, int q_head, int q_offset,
                                        T* __restrict__ out, int out_head, int out_offset, int heads, int rot,
-                                       int rot_dims, const int* __restrict__ positions,
+                                       int rot_dims, float amplitude, const int* __restrict__ positions,
                                        const float* __restrict__ inv_freq, long long total) {
   const int half = rot_dims / 2;
   const int per_head = rot - half;       // `half` pairs, then the dims that pass unchanged
@@ -77,8 +102,8 @@ __global__ void latent_q_rotate_kernel(const T* __restrict__ q, long long ldq, i
     float sn, cs;
     sincosf((float)positions[t] * inv_freq[i], &sn, &cs);
     const float lo = to_float<T>(src[i]), hi = to_float<T>(src[i + half]);
-    dst[i] = from_float<T>(lo * cs - hi * sn);
-    dst[i + half] = from_float<T>(hi * cs + lo * sn);
+    dst[i] = from_float<T>(amplitude * (lo * cs - hi * sn));
+    dst[i + half] = from_float<T>(amplitude * (hi * cs + lo * sn));
   } else {
     dst[i + half] = src[i + half];
   }
@@ -88,11 +113,17 @@ __global__ void latent_q_rotate_kernel(const T* __restrict__ q, long long ldq, i
 // A product per head: out[t, h, n] = sum_k a[t, h, k] * w[h, n, k].  a: row stride lda, head stride sa; out: row
 // stride ldo, head stride so; w contiguous [heads, N, K].  Grid (ceil(T / 64), ceil(N / 64), heads), 256 threads,
 // each 4 x 4 outputs; K in steps of 16 through LDS; an output element is one FMA chain in k order, so it does not
-// depend on the other rows of the launch.
+// depend on the other rows of the launch.  gate [T, ldg] 32-bit (null: none): the outputs of head h are multiplied by
+// sigmoid(gate[t, h]).
+__device__ __forceinline__ float head_gate(const float* gate, long long ldg, int t, int h) {
+  return gate ? 1.0f / (1.0f + expf(-gate[(long long)t * ldg + h])) : 1.0f;
+}
+
 template <typename TA, typename TW, typename TO>
 __global__ __launch_bounds__(256) void head_linear_kernel(const TA* __restrict__ a, long long lda, long long sa,
                                                           const TW* __restrict__ w, TO* __restrict__ out,
-                                                          long long ldo, long long so, int M, int N, int K) {
+                                                          long long ldo, long long so, int M, int N, int K,
+                                                          const float* __restrict__ gate, long long ldg) {
   __shared__ float As[16][64 + 4];
   __shared__ float Ws[16][64 + 4];
   const int h = blockIdx.z;
@@ -127,10 +158,11 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const TA* __restrict__
   for (int i = 0; i < 4; ++i) {
     const int m = m0 + ty * 4 + i;
     if (m >= M) continue;
+    const float open = head_gate(gate, ldg, m, h);
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
-      if (n < N) out[(long long)m * ldo + (long long)h * so + n] = from_float<TO>(acc[i][j]);
+      if (n < N) out[(long long)m * ldo + (long long)h * so + n] = from_float<TO>(acc[i][j] * open);
     }
   }
 }
@@ -139,7 +171,8 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const TA* __restrict__
 // x 128 outputs of one head, see group_tile.h.  Grid (ceil(T / 128), ceil(N / 128), heads).
 __global__ __launch_bounds__(256) void head_linear_mma_kernel(const __bf16* __restrict__ a, long long lda, long long sa,
                                                               const __bf16* __restrict__ w, __bf16* __restrict__ out,
-                                                              long long ldo, long long so, int M, int N, int K) {
+                                                              long long ldo, long long so, int M, int N, int K,
+                                                              const float* __restrict__ gate, long long ldg) {
   extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
   const int h = blockIdx.z, m0 = blockIdx.x * GT_TILE, n0 = blockIdx.y * GT_TILE;
   const __bf16* ah = a + (long long)h * sa;
@@ -154,33 +187,39 @@ __global__ __launch_bounds__(256) void head_linear_mma_kernel(const __bf16* __re
     const int m = m0 + wm * 64 + tm * 16 + lr;
     if (m >= M) continue;
     __bf16* dst = out + (long long)m * ldo + (long long)h * so;
+    const float open = head_gate(gate, ldg, m, h);
 #pragma unroll
     for (int tn = 0; tn < 4; ++tn)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int n = n0 + wn * 64 + tn * 16 + lg * 4 + i;
-        if (n < N) dst[n] = (__bf16)acc[tn][tm][i];
+        if (n < N) dst[n] = (__bf16)(acc[tn][tm][i] * open);
       }
   }
 }
 
 // ---------------------------------------------------------------------------------------------
-extern "C" int vk_latent_kv_write(const float* x, long long ldx, const float* weight, float eps, int rank, int rot,
-                                  int rot_dims, const int* positions, const float* inv_freq, const int* entry_of,
-                                  const int* table, int table_width, int block_size, void* k_cache, void* v_cache,
-                                  int cache_dtype, int num_tokens, void* stream) {
+extern "C" int vk_latent_prepare(const float* x, const float* xq, long long ldx, const float* weight, float eps, int rank,
+                                 int rot, int rot_dims, float amplitude, const int* positions, const float* inv_freq,
+                                 const int* entry_of, const int* table, int table_width, int block_size, void* k_cache,
+                                 void* v_cache, const float* q_weight, int q_rank, void* q_out, int dtype, int num_tokens,
+                                 void* stream) {
   if (num_tokens <= 0) return 0;
-  if (rank < 1 || rot < 0 || rot_dims < 0 || rot_dims > rot || (rot_dims & 1) || block_size < 1 || table_width < 1)
+  if (k_cache && (rank < 1 || rot < 0 || rot_dims < 0 || rot_dims > rot || (rot_dims & 1) || block_size < 1 || table_width < 1 ||
+                  !x || !weight || !v_cache || !positions || !entry_of || !table || (rot_dims && !inv_freq)))
     return VK_BAD_ARGUMENT;
+  if (q_out && (q_rank < 1 || !xq || !q_weight)) return VK_BAD_ARGUMENT;
+  if (!k_cache && !q_out) return 0;
   hipStream_t s = (hipStream_t)stream;
-  if (cache_dtype == DT_F32)
-    latent_kv_write_kernel<float><<<num_tokens, 256, 0, s>>>(x, ldx, weight, eps, rank, rot, rot_dims, positions,
+  if (dtype == DT_F32)
+    latent_prepare_kernel<float><<<num_tokens, 256, 0, s>>>(x, xq, ldx, weight, eps, rank, rot, rot_dims, amplitude, positions,
+                                                            inv_freq, entry_of, table, table_width, block_size, (float*)k_cache,
+                                                            (float*)v_cache, q_weight, q_rank, (float*)q_out);
+  else if (dtype == DT_BF16)
+    latent_prepare_kernel<bf16_t><<<num_tokens, 256, 0, s>>>(x, xq, ldx, weight, eps, rank, rot, rot_dims, amplitude, positions,
                                                              inv_freq, entry_of, table, table_width, block_size,
-                                                             (float*)k_cache, (float*)v_cache);
-  else if (cache_dtype == DT_BF16)
-    latent_kv_write_kernel<bf16_t><<<num_tokens, 256, 0, s>>>(x, ldx, weight, eps, rank, rot, rot_dims, positions,
-                                                              inv_freq, entry_of, table, table_width, block_size,
-                                                              (bf16_t*)k_cache, (bf16_t*)v_cache);
+                                                             (bf16_t*)k_cache, (bf16_t*)v_cache, q_weight, q_rank,
+                                                             (bf16_t*)q_out);
   else
     return VK_BAD_ARGUMENT;
   VK_LAUNCH_CHECK();
@@ -188,7 +227,7 @@ extern "C" int vk_latent_kv_write(const float* x, long long ldx, const float* we
 }
 
 extern "C" int vk_latent_q_rotate(const void* q, long long ldq, int q_head, int q_offset, void* out, int out_head,
-                                  int out_offset, int heads, int rot, int rot_dims, const int* positions,
+                                  int out_offset, int heads, int rot, int rot_dims, float amplitude, const int* positions,
                                   const float* inv_freq, int dtype, int num_tokens, void* stream) {
   if (num_tokens <= 0 || rot <= 0) return 0;
   if (heads < 1 || rot_dims < 0 || rot_dims > rot || (rot_dims & 1)) return VK_BAD_ARGUMENT;
@@ -197,10 +236,10 @@ extern "C" int vk_latent_q_rotate(const void* q, long long ldq, int q_head, int 
   hipStream_t s = (hipStream_t)stream;
   if (dtype == DT_F32)
     latent_q_rotate_kernel<float><<<blocks, 256, 0, s>>>((const float*)q, ldq, q_head, q_offset, (float*)out, out_head,
-                                                         out_offset, heads, rot, rot_dims, positions, inv_freq, total);
+                                                         out_offset, heads, rot, rot_dims, amplitude, positions, inv_freq, total);
   else if (dtype == DT_BF16)
     latent_q_rotate_kernel<bf16_t><<<blocks, 256, 0, s>>>((const bf16_t*)q, ldq, q_head, q_offset, (bf16_t*)out,
-                                                          out_head, out_offset, heads, rot, rot_dims, positions,
+                                                          out_head, out_offset, heads, rot, rot_dims, amplitude, positions,
                                                           inv_freq, total);
   else
     return VK_BAD_ARGUMENT;
@@ -210,7 +249,7 @@ extern "C" int vk_latent_q_rotate(const void* q, long long ldq, int q_head, int 
 
 extern "C" int vk_head_linear(const void* a, int a_dtype, long long lda, long long sa, const void* w, int w_dtype,
                               void* out, int out_dtype, long long ldo, long long so, int M, int N, int K, int heads,
-                              void* stream) {
+                              const float* gate, long long ldg, void* stream) {
   if (M <= 0 || N <= 0 || heads <= 0) return 0;
   if (K < 1 || heads > 65535) return VK_BAD_ARGUMENT;
   dim3 grid((M + 63) / 64, (N + 63) / 64, heads);
@@ -218,7 +257,7 @@ extern "C" int vk_head_linear(const void* a, int a_dtype, long long lda, long lo
   hipStream_t s = (hipStream_t)stream;
   if (a_dtype == DT_F32 && w_dtype == DT_F32 && out_dtype == DT_F32)
     head_linear_kernel<float, float, float><<<grid, 256, 0, s>>>((const float*)a, lda, sa, (const float*)w, (float*)out,
-                                                                 ldo, so, M, N, K);
+                                                                 ldo, so, M, N, K, gate, ldg);
   else if (a_dtype == DT_BF16 && w_dtype == DT_BF16 && out_dtype == DT_BF16 && K % 8 == 0 && lda % 8 == 0 && sa % 8 == 0 &&
            (((uintptr_t)a | (uintptr_t)w) & 15) == 0) {
     static bool sized = false;
@@ -230,13 +269,13 @@ extern "C" int vk_head_linear(const void* a, int a_dtype, long long lda, long lo
     }
     dim3 wide((M + GT_TILE - 1) / GT_TILE, (N + GT_TILE - 1) / GT_TILE, heads);
     head_linear_mma_kernel<<<wide, 256, GT_LDS_BYTES, s>>>((const __bf16*)a, lda, sa, (const __bf16*)w, (__bf16*)out, ldo,
-                                                           so, M, N, K);
+                                                           so, M, N, K, gate, ldg);
   } else if (a_dtype == DT_BF16 && w_dtype == DT_BF16 && out_dtype == DT_BF16)
     head_linear_kernel<bf16_t, bf16_t, bf16_t><<<grid, 256, 0, s>>>((const bf16_t*)a, lda, sa, (const bf16_t*)w,
-                                                                    (bf16_t*)out, ldo, so, M, N, K);
+                                                                    (bf16_t*)out, ldo, so, M, N, K, gate, ldg);
   else if (a_dtype == DT_BF16 && w_dtype == DT_F32 && out_dtype == DT_BF16)
     head_linear_kernel<bf16_t, float, bf16_t><<<grid, 256, 0, s>>>((const bf16_t*)a, lda, sa, (const float*)w,
-                                                                   (bf16_t*)out, ldo, so, M, N, K);
+                                                                   (bf16_t*)out, ldo, so, M, N, K, gate, ldg);
   else
     return VK_BAD_ARGUMENT;
   VK_LAUNCH_CHECK();

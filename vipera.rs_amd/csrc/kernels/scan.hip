@@ -280,6 +280,40 @@ __global__ __launch_bounds__(256) void conv_keep_kernel(const float* __restrict_
   }
 }
 
+// Both at once where every entry is a single token (one token per entry, so entry e is token entry_start[e]): a thread
+// owns a channel, takes its old inputs in order and moves each one place down as it has used it.  The sum's order is
+// causal_conv_kernel's.
+template <typename TO>
+__global__ __launch_bounds__(256) void causal_conv_single_kernel(const float* __restrict__ in, long long ldi,
+                                                                 const float* __restrict__ conv,
+                                                                 const float* __restrict__ bias, int taps, int C,
+                                                                 float* __restrict__ state, long long state_stride,
+                                                                 long long conv_offset,
+                                                                 const int* __restrict__ entry_start,
+                                                                 const int* __restrict__ entry_first,
+                                                                 const int* __restrict__ slots, float* __restrict__ y32,
+                                                                 TO* __restrict__ yrun) {
+  const int e = blockIdx.x;
+  const int c = blockIdx.y * 256 + threadIdx.x;
+  if (c >= C) return;
+  const int t = entry_start[e];
+  const bool fresh = entry_first[e] == 0;
+  float* rows = state + (long long)slots[e] * state_stride + conv_offset + c;
+  const float now = in[(long long)t * ldi + c];
+  float sum = bias ? bias[c] : 0.f;
+  for (int j = 0; j + 1 < taps; ++j) {
+    const float old = rows[(long long)j * C];
+    const float x = fresh ? 0.f : old;
+    sum = fmaf(conv[(long long)c * taps + j], x, sum);
+    if (j > 0) rows[(long long)(j - 1) * C] = x;
+  }
+  sum = fmaf(conv[(long long)c * taps + taps - 1], now, sum);
+  if (taps > 1) rows[(long long)(taps - 2) * C] = now;
+  const float y = scan_silu(sum);
+  y32[(long long)t * C + c] = y;
+  if (yrun) yrun[(long long)t * C + c] = from_float<TO>(y);
+}
+
 extern "C" int vk_causal_conv(const float* in, long long ldi, const float* conv, const float* bias, int taps, int C,
                               float* state, long long state_stride, long long conv_offset, const int* entry_of,
                               const int* entry_start, const int* entry_first, const int* slots, int num_tokens,
@@ -289,6 +323,19 @@ extern "C" int vk_causal_conv(const float* in, long long ldi, const float* conv,
   dim3 grid(num_tokens, (C + 255) / 256);
   if (grid.y > 65535) return VK_UNSUPPORTED_SIZE;
   hipStream_t s = (hipStream_t)stream;
+  if (num_tokens == num_entries) {
+    dim3 singles(num_entries, grid.y);
+    if (yrun == nullptr || run_dtype == DT_F32)
+      causal_conv_single_kernel<float><<<singles, 256, 0, s>>>(in, ldi, conv, bias, taps, C, state, state_stride, conv_offset,
+                                                               entry_start, entry_first, slots, y32, (float*)yrun);
+    else if (run_dtype == DT_BF16)
+      causal_conv_single_kernel<bf16_t><<<singles, 256, 0, s>>>(in, ldi, conv, bias, taps, C, state, state_stride, conv_offset,
+                                                                entry_start, entry_first, slots, y32, (bf16_t*)yrun);
+    else
+      return VK_BAD_ARGUMENT;
+    VK_LAUNCH_CHECK();
+    return 0;
+  }
   if (yrun == nullptr || run_dtype == DT_F32)
     causal_conv_kernel<float><<<grid, 256, 0, s>>>(in, ldi, conv, bias, taps, C, state, state_stride, conv_offset,
                                                    entry_of, entry_start, entry_first, slots, y32, (float*)yrun);

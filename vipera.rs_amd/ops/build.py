@@ -38,6 +38,8 @@ MODULES: Dict[str, tuple] = {
     "sampling": ("hip", ["kernels/sampling.hip"], ["kernels/common.h"]),
     "recurrent": ("hip", ["kernels/recurrent.hip"], ["kernels/common.h"]),
     "scan": ("hip", ["kernels/scan.hip"], ["kernels/common.h"]),
+    "state_space": ("hip", ["kernels/state_space.hip"], ["kernels/common.h"]),
+    "streams": ("hip", ["kernels/streams.hip"], ["kernels/common.h"]),
     "latent": ("hip", ["kernels/latent.hip"], ["kernels/common.h", "kernels/group_tile.h"]),
     "moe": ("hip", ["kernels/moe.hip"], ["kernels/common.h", "kernels/group_tile.h"]),
     "host": ("host", ["host/cache_manager.cpp", "host/scheduler.cpp", "host/c_api.cpp"],

@@ -111,8 +111,9 @@ def fetch_words(pinned: torch.Tensor, out: torch.Tensor) -> bool:
 
 # ----------------------------------------------------------------------------------------------
 def embed_gather(table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor,
-                 source: Optional[torch.Tensor] = None, sampled: Optional[torch.Tensor] = None) -> None:
-    """``out[t, :] = table[tokens[t], :]`` widened to 32-bit.  The caller has checked the ids.
+                 source: Optional[torch.Tensor] = None, sampled: Optional[torch.Tensor] = None,
+                 scale: float = 1.0) -> None:
+    """``out[t, :] = table[tokens[t], :] * scale`` in 32-bit.  The caller has checked the ids.
 
     With ``source`` and ``sampled``: where ``source[t] >= 0`` the id is ``sampled[source[t]]``, which an
     earlier kernel of the stream left on the device."""
@@ -126,9 +127,9 @@ def embed_gather(table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor,
               "embed_gather: sampled must be contiguous int32")
         _need(source.dtype == torch.int32 and source.numel() >= num_tokens and source.is_contiguous(),
               "embed_gather: source")
-    fn = _fn("elementwise", "vk_embed_gather", [_p, _i, _p, _p, _p, _p, _i, _i, _i, _p])
+    fn = _fn("elementwise", "vk_embed_gather_scaled", [_p, _i, _p, _p, _p, _p, _i, _i, _i, _f, _p])
     _status(fn(_ptr(table), _dt(table, "table"), _ptr(tokens), _ptr(source), _ptr(sampled if source is not None else None),
-               _ptr(out), num_tokens, width, table.shape[0], _stream()), "embed_gather")
+               _ptr(out), num_tokens, width, table.shape[0], float(scale), _stream()), "embed_gather")
 
 
 def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor,
@@ -148,15 +149,16 @@ def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor
             "rmsnorm")
 
 
-def rope_angles(positions: torch.Tensor, inv_freq: torch.Tensor, num_tokens: int) -> torch.Tensor:
+def rope_angles(positions: torch.Tensor, inv_freq: torch.Tensor, num_tokens: int, amplitude: float = 1.0) -> torch.Tensor:
     """``[num_tokens, len(inv_freq), 2]`` floats: sine and cosine of ``float(pos) * inv_freq`` for a step's
-    tokens, computed once where many heads and layers would each compute them again."""
+    tokens, times ``amplitude``, computed once where many heads and layers would each compute them again."""
     _dev(positions, inv_freq)
     _need(positions.dtype == torch.int32 and positions.numel() >= num_tokens, "rope_angles: positions")
     _need(inv_freq.dtype == torch.float32 and inv_freq.is_contiguous(), "rope_angles: inv_freq must be float32")
     out = torch.empty((num_tokens, inv_freq.numel(), 2), dtype=torch.float32, device=positions.device)
-    fn = _fn("elementwise", "vk_rope_angles", [_p, _p, _i, _i, _p, _p])
-    _status(fn(_ptr(positions), _ptr(inv_freq), inv_freq.numel(), num_tokens, _ptr(out), _stream()), "rope_angles")
+    fn = _fn("elementwise", "vk_rope_angles_scaled", [_p, _p, _i, _i, _f, _p, _p])
+    _status(fn(_ptr(positions), _ptr(inv_freq), inv_freq.numel(), num_tokens, float(amplitude), _ptr(out), _stream()),
+            "rope_angles")
     return out
 
 
@@ -1211,30 +1213,51 @@ def head_norm_gate(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, ga
 
 
 # --- latent attention -----------------------------------------------------------------------------
-def latent_kv_write(x: torch.Tensor, weight: torch.Tensor, eps: float, rank: int, rot: int, rot_dims: int,
-                    positions: torch.Tensor, inv_freq: Optional[torch.Tensor], entry_of: torch.Tensor,
-                    table: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor) -> None:
-    """A step's cached rows ``[rms_norm(x[:rank]) * weight | rotate(x[rank:rank + rot])]`` into their pages, as keys
-    and transposed as values (one key head of width ``rank + rot``).  ``x``: a 32-bit row-strided view."""
-    _dev(x, weight, positions, inv_freq, entry_of, table, k_cache, v_cache)
-    tokens = x.shape[0]
+def latent_prepare(x: Optional[torch.Tensor], weight: Optional[torch.Tensor], eps: float, rank: int, rot: int, rot_dims: int,
+                   positions: torch.Tensor, inv_freq: Optional[torch.Tensor], entry_of: torch.Tensor,
+                   table: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, amplitude: float = 1.0,
+                   x_q: Optional[torch.Tensor] = None, q_weight: Optional[torch.Tensor] = None,
+                   q_out: Optional[torch.Tensor] = None) -> None:
+    """What follows a step's down products, in one launch.  ``x`` (a 32-bit row-strided view, or None: a layer that keeps
+    no rows): the cached rows ``[rms_norm(x[:rank]) * weight | rotate(x[rank:rank + rot])]`` go into their pages, as keys
+    and transposed as values (one key head of width ``rank + rot``); sines and cosines are multiplied by ``amplitude``.
+    ``q_out``: the queries' latent ``rms_norm(x_q) * q_weight``, ``x_q`` a view with ``x``'s row stride."""
+    _dev(x, weight, positions, inv_freq, entry_of, table, k_cache, v_cache, x_q, q_weight, q_out)
+    _need(x is not None or q_out is not None, "latent_prepare: nothing to do")
+    tokens = (x if x is not None else x_q).shape[0]
+    stride = (x if x is not None else x_q).stride(0)
     width = rank + rot
-    _need(x.dim() == 2 and x.dtype == torch.float32 and x.stride(1) == 1 and x.shape[1] == width, "latent_kv_write: x")
-    _need(weight.dtype == torch.float32 and weight.numel() == rank and weight.is_contiguous(), "latent_kv_write: weight")
-    _need(_cache_ok(k_cache, v_cache, 1, width, k_cache.dtype), "latent_kv_write: cache shape")
-    _i32(positions, entry_of, table)
-    _need(positions.numel() >= tokens and entry_of.numel() >= tokens and table.dim() == 2, "latent_kv_write: indices")
-    _need(rot_dims == 0 or (inv_freq is not None and inv_freq.dtype == torch.float32 and inv_freq.numel() == rot_dims // 2),
-          "latent_kv_write: inv_freq")
-    fn = _fn("latent", "vk_latent_kv_write", [_p, _ll, _p, _f, _i, _i, _i, _p, _p, _p, _p, _i, _i, _p, _p, _i, _i, _p])
-    _status(fn(_ptr(x), x.stride(0), _ptr(weight), float(eps), rank, rot, rot_dims, _ptr(positions), _ptr(inv_freq),
-               _ptr(entry_of), _ptr(table), table.shape[1], k_cache.shape[2], _ptr(k_cache), _ptr(v_cache),
-               _dt(k_cache, "cache"), tokens, _stream()), "latent_kv_write")
+    if x is not None:
+        _need(x.dim() == 2 and x.dtype == torch.float32 and x.stride(1) == 1 and x.shape[1] == width, "latent_prepare: x")
+        _need(weight is not None and weight.dtype == torch.float32 and weight.numel() == rank and weight.is_contiguous(),
+              "latent_prepare: weight")
+        _need(_cache_ok(k_cache, v_cache, 1, width, k_cache.dtype), "latent_prepare: cache shape")
+        _i32(positions, entry_of, table)
+        _need(positions.numel() >= tokens and entry_of.numel() >= tokens and table.dim() == 2, "latent_prepare: indices")
+        _need(rot_dims == 0 or (inv_freq is not None and inv_freq.dtype == torch.float32
+                                and inv_freq.numel() == rot_dims // 2), "latent_prepare: inv_freq")
+    q_rank = 0
+    if q_out is not None:
+        q_rank = q_out.shape[1]
+        _need(x_q is not None and x_q.dtype == torch.float32 and x_q.shape == (tokens, q_rank) and x_q.stride(1) == 1
+              and (x_q.stride(0) == stride or tokens == 1) and q_out.shape[0] == tokens and q_out.is_contiguous()
+              and q_out.dtype == k_cache.dtype, "latent_prepare: x_q and q_out")
+        _need(q_weight is not None and q_weight.dtype == torch.float32 and q_weight.numel() == q_rank
+              and q_weight.is_contiguous(), "latent_prepare: q_weight")
+    keeps = x is not None
+    fn = _fn("latent", "vk_latent_prepare", [_p, _p, _ll, _p, _f, _i, _i, _i, _f, _p, _p, _p, _p, _i, _i, _p, _p, _p, _i, _p,
+                                             _i, _i, _p])
+    _status(fn(_ptr(x), _ptr(x_q), stride, _ptr(weight), float(eps), rank, rot, rot_dims, float(amplitude), _ptr(positions),
+               _ptr(inv_freq), _ptr(entry_of), _ptr(table), table.shape[1], k_cache.shape[2],
+               _ptr(k_cache if keeps else None), _ptr(v_cache if keeps else None), _ptr(q_weight), q_rank, _ptr(q_out),
+               _dt(k_cache, "cache"), tokens, _stream()), "latent_prepare")
 
 
 def latent_q_rotate(q: torch.Tensor, q_head: int, q_offset: int, out: torch.Tensor, out_head: int, out_offset: int,
-                    heads: int, rot: int, rot_dims: int, positions: torch.Tensor, inv_freq: Optional[torch.Tensor]) -> None:
-    """``out[t, h, out_offset:out_offset + rot] = rotate(q[t, h, q_offset:q_offset + rot])`` for every head."""
+                    heads: int, rot: int, rot_dims: int, positions: torch.Tensor, inv_freq: Optional[torch.Tensor],
+                    amplitude: float = 1.0) -> None:
+    """``out[t, h, out_offset:out_offset + rot] = rotate(q[t, h, q_offset:q_offset + rot])`` for every head; sines and
+    cosines are multiplied by ``amplitude``."""
     _dev(q, out, positions, inv_freq)
     tokens = q.shape[0]
     _need(q.dim() == 2 and q.stride(1) == 1 and q.shape[1] >= heads * q_head and q_offset + rot <= q_head, "latent_q_rotate: q")
@@ -1243,24 +1266,29 @@ def latent_q_rotate(q: torch.Tensor, q_head: int, q_offset: int, out: torch.Tens
     _i32(positions)
     _need(rot_dims == 0 or (inv_freq is not None and inv_freq.dtype == torch.float32 and inv_freq.numel() == rot_dims // 2),
           "latent_q_rotate: inv_freq")
-    fn = _fn("latent", "vk_latent_q_rotate", [_p, _ll, _i, _i, _p, _i, _i, _i, _i, _i, _p, _p, _i, _i, _p])
+    fn = _fn("latent", "vk_latent_q_rotate", [_p, _ll, _i, _i, _p, _i, _i, _i, _i, _i, _f, _p, _p, _i, _i, _p])
     _status(fn(_ptr(q), q.stride(0), q_head, q_offset, _ptr(out), out_head, out_offset, heads, rot, rot_dims,
-               _ptr(positions), _ptr(inv_freq), _dt(q, "q"), tokens, _stream()), "latent_q_rotate")
+               float(amplitude), _ptr(positions), _ptr(inv_freq), _dt(q, "q"), tokens, _stream()), "latent_q_rotate")
 
 
 def head_linear(a: torch.Tensor, a_head_stride: int, k: int, w: torch.Tensor, out: torch.Tensor,
-                out_head_stride: int) -> None:
-    """A product per head: ``out[t, h*so : h*so + N] = w[h] @ a[t, h*sa : h*sa + K]``; ``w``: ``[heads, N, K]``."""
-    _dev(a, w, out)
+                out_head_stride: int, gate: Optional[torch.Tensor] = None) -> None:
+    """A product per head: ``out[t, h*so : h*so + N] = w[h] @ a[t, h*sa : h*sa + K]``; ``w``: ``[heads, N, K]``.  ``gate`` (a
+    32-bit row-strided view ``[T, heads]``): head ``h``'s outputs are multiplied by ``sigmoid(gate[t, h])``."""
+    _dev(a, w, out, gate)
     heads, n, kw = w.shape
     tokens = a.shape[0]
     _need(kw == k and w.is_contiguous(), "head_linear: w")
     _need(a.dim() == 2 and a.stride(1) == 1 and (heads - 1) * a_head_stride + k <= a.shape[1], "head_linear: a")
     _need(out.dim() == 2 and out.stride(1) == 1 and out.shape[0] == tokens
           and (heads - 1) * out_head_stride + n <= out.shape[1], "head_linear: out")
-    fn = _fn("latent", "vk_head_linear", [_p, _i, _ll, _ll, _p, _i, _p, _i, _ll, _ll, _i, _i, _i, _i, _p])
+    if gate is not None:
+        _need(gate.dtype == torch.float32 and gate.shape == (tokens, heads) and (gate.stride(1) == 1 or heads == 1),
+              "head_linear: gate")
+    fn = _fn("latent", "vk_head_linear", [_p, _i, _ll, _ll, _p, _i, _p, _i, _ll, _ll, _i, _i, _i, _i, _p, _ll, _p])
     _status(fn(_ptr(a), _dt(a, "a"), a.stride(0), a_head_stride, _ptr(w), _dt(w, "w"), _ptr(out), _dt(out, "out"),
-               out.stride(0), out_head_stride, tokens, n, k, heads, _stream()), "head_linear")
+               out.stride(0), out_head_stride, tokens, n, k, heads, _ptr(gate), gate.stride(0) if gate is not None else 0,
+               _stream()), "head_linear")
 
 
 # --- mixture of experts ---------------------------------------------------------------------------
@@ -1618,10 +1646,11 @@ def head_prepare(proj: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight:
                  norm_first: bool, eps: float, positions: Optional[torch.Tensor], inv_freq: Optional[torch.Tensor],
                  rot_dims: int, heads: int, kv_heads: int, maps: int, dim: int, vdim: int, width: int,
                  qkv: torch.Tensor, k_cache: Optional[torch.Tensor] = None, v_cache: Optional[torch.Tensor] = None,
-                 entry_of_token: Optional[torch.Tensor] = None, block_table: Optional[torch.Tensor] = None) -> None:
+                 entry_of_token: Optional[torch.Tensor] = None, block_table: Optional[torch.Tensor] = None,
+                 amplitude: float = 1.0) -> None:
     """The 32-bit sums ``proj`` = ``[q | k | v | ...]`` of a step's tokens laid out head by head at one padded
-    ``width`` in ``qkv``: q and k heads rotated by position (the first ``rot_dims`` numbers, half-split pairs) and, with
-    ``norm``, divided by their root mean square and multiplied by a weight of ``dim`` numbers (None: no weight), before
+    ``width`` in ``qkv``: q and k heads rotated by position (the first ``rot_dims`` numbers, half-split pairs, sines and cosines times
+    ``amplitude``) and, with ``norm``, divided by their root mean square and multiplied by a weight of ``dim`` numbers (None: no weight), before
     the rotation (``norm_first``) or behind it.  ``maps`` > 1: that many attention maps per head; a query head's maps
     become query heads of their own, each in its own columns of the padded width, and a key head's maps stay side by
     side in one key head, so every map meets its own keys and all maps of a head read the same values.  With
@@ -1651,11 +1680,11 @@ def head_prepare(proj: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight:
         _need(entry_of_token.dtype == torch.int32 and entry_of_token.numel() >= tokens and positions.dtype == torch.int32
               and positions.numel() >= tokens, "head_prepare: entries and positions")
         table_width, block_size = block_table.shape[1], k_cache.shape[2]
-    fn = _fn("heads", "vk_head_prepare", [_p, _ll, _p, _p, _i, _i, _f, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _p, _i,
+    fn = _fn("heads", "vk_head_prepare", [_p, _ll, _p, _p, _i, _i, _f, _p, _p, _i, _f, _i, _i, _i, _i, _i, _i, _i, _p, _i,
                                           _p, _p, _p, _p, _i, _i, _p])
     _status(fn(_ptr(proj), proj.stride(0), _ptr(q_weight), _ptr(k_weight), 1 if norm else 0, 1 if norm_first else 0,
-               float(eps), _ptr(positions), _ptr(inv_freq), int(rot_dims), tokens, heads, kv_heads, maps, dim, vdim,
-               width, _ptr(qkv), _dt(qkv, "qkv"), _ptr(k_cache), _ptr(v_cache), _ptr(entry_of_token), _ptr(block_table),
+               float(eps), _ptr(positions), _ptr(inv_freq), int(rot_dims), float(amplitude), tokens, heads, kv_heads, maps, dim,
+               vdim, width, _ptr(qkv), _dt(qkv, "qkv"), _ptr(k_cache), _ptr(v_cache), _ptr(entry_of_token), _ptr(block_table),
                table_width, block_size, _stream()), "head_prepare")
 
 
@@ -1709,3 +1738,123 @@ def row_gate_add(y: torch.Tensor, gate: torch.Tensor, gate_kind: str, out: torch
     fn = _fn("heads", "vk_row_gate_add", [_p, _p, _ll, _i, _p, _i, _i, _i, _p])
     _status(fn(_ptr(y), _ptr(gate), gate.stride(0), _GATE_ACTS[gate_kind], _ptr(out), y.shape[0], y.shape[1],
                1 if accumulate else 0, _stream()), "row_gate_add")
+
+
+# --- residual streams -------------------------------------------------------------------------------
+STREAMS_MAX = 8
+STREAMS_MAX_WIDTH = 16_384     # a row stays in a workgroup's registers between its sums and its norm
+STREAM_NORMS = {"none": 0, "rms": 1, "layer": 2}
+
+
+def streams_step(src: torch.Tensor, streams: int, y: Optional[torch.Tensor], mix: Optional[torch.Tensor],
+                 share: Optional[torch.Tensor], dst: Optional[torch.Tensor], read: Optional[torch.Tensor],
+                 out: Optional[torch.Tensor], norm: str = "none", weight: Optional[torch.Tensor] = None,
+                 bias: Optional[torch.Tensor] = None, eps: float = 0.0, rows: Optional[torch.Tensor] = None) -> None:
+    """The end of one sublayer and the beginning of the next over a token's ``streams`` residual streams, in 32-bit.
+
+    ``src``: ``[tokens, streams, width]``, or ``[tokens, width]`` where all streams still are that row.  ``y`` (``[tokens,
+    width]`` with ``mix [streams, streams]`` and ``share [streams]``): the streams become ``sum_s mix[s, t] x_s + share[t]
+    y``, which ``dst`` receives if it is given (it may be ``src``).  ``out``: ``norm(sum_s read[s] x_s)`` of the new streams
+    (``read`` None: the plain sum), of the tokens in ``rows`` (None: all); ``norm``: ``none``, ``rms`` or ``layer`` with
+    ``weight`` and ``bias``."""
+    _dev(src, y, mix, share, dst, read, out, weight, bias, rows)
+    tokens, width = src.shape[0], src.shape[-1]
+    _f32(src, "streams_step: src")
+    _need(src.shape in ((tokens, width), (tokens, streams, width)), "streams_step: src shape")
+    if streams > STREAMS_MAX:
+        raise UnsupportedError(f"streams_step: {streams} streams are above the kernel's limit of {STREAMS_MAX}")
+    if y is not None:
+        _need(mix is not None and share is not None, "streams_step: an output joins through mix and share")
+        for t, shape, what in ((y, (tokens, width), "y"), (mix, (streams, streams), "mix"), (share, (streams,), "share")):
+            _f32(t, "streams_step: " + what)
+            _need(t.shape == shape, f"streams_step: {what} shape")
+    if dst is not None:
+        _f32(dst, "streams_step: dst")
+        _need(y is not None and rows is None and dst.shape == (tokens, streams, width), "streams_step: dst")
+        _need(dst.data_ptr() != src.data_ptr() or src.dim() == 3, "streams_step: dst may be src only where src holds streams")
+    if width > STREAMS_MAX_WIDTH:
+        raise UnsupportedError(f"streams_step: a width of {width} is above the kernel's limit of {STREAMS_MAX_WIDTH}")
+    count = tokens if rows is None else rows.numel()
+    if rows is not None:
+        _i32(rows)
+    if read is not None:
+        _need(read.dtype == torch.float32 and read.numel() == streams and read.is_contiguous(), "streams_step: read")
+    if out is not None:
+        _need(out.shape == (count, width) and out.is_contiguous(), "streams_step: out shape")
+    for t, what in ((weight, "weight"), (bias, "bias")):
+        if t is not None:
+            _need(t.dtype == torch.float32 and t.numel() == width and t.is_contiguous(), f"streams_step: {what}")
+    _need(norm in STREAM_NORMS, "streams_step: norm")
+    held = src.dim() == 3
+    fn = _fn("streams", "vk_streams_step", [_p, _ll, _ll, _p, _p, _p, _p, _p, _i, _p, _p, _f, _p, _p, _i, _i, _i, _i, _p])
+    _status(fn(_ptr(src), streams * width if held else width, width if held else 0, _ptr(y), _ptr(mix), _ptr(share),
+               _ptr(dst), _ptr(read), STREAM_NORMS[norm], _ptr(weight), _ptr(bias), float(eps), _ptr(rows), _ptr(out),
+               _dt(out, "out") if out is not None else 0, count, streams, width, _stream()), "streams_step")
+
+
+# --- state-space recurrence ---------------------------------------------------------------------------
+STATE_SPACE_MAX_STATES = 256
+STATE_SPACE_CHUNK = 64        # tokens of a chunk of the chunked form
+STATE_SPACE_STEP_TOKENS = 6   # entries of up to this many tokens go token by token
+
+
+def state_space_head_floats(vdim: int, states: int) -> int:
+    """32-bit numbers of one head's state in a slot's row."""
+    return vdim * ((states + 3) // 4 * 4)
+
+
+def state_space(x: torch.Tensor, b: torch.Tensor, c: torch.Tensor, dt: torch.Tensor, dt_bias: torch.Tensor,
+                a_log: torch.Tensor, skip: torch.Tensor, state: torch.Tensor, entry_start: torch.Tensor,
+                entry_first_pos: torch.Tensor, slots: torch.Tensor, heads: int, groups: int, vdim: int, states: int,
+                out: torch.Tensor, num_entries: int, min_count: int, max_count: int,
+                step_tokens: int = STATE_SPACE_STEP_TOKENS) -> None:
+    """The state-space recurrence with one decay per head and token over the step's entries, in 32-bit: per head
+    ``d = softplus(dt + dt_bias); S <- exp(-exp(a_log) d) S + d b x^T; y = S^T c + skip x`` (``S`` is ``states x vdim``;
+    head ``h`` reads group ``h // (heads / groups)`` of ``b`` and ``c``).  ``x [T, heads * vdim]``, ``b``, ``c [T, groups *
+    states]``: row-strided 32-bit views with one stride; ``dt [T, heads]`` a row-strided 32-bit view.  ``state [slots + 1,
+    floats]`` starts with ``heads * state_space_head_floats(vdim, states)`` floats of this layer.  ``min_count`` and
+    ``max_count``: tokens of the shortest and the longest entry; entries of more than ``step_tokens`` run in chunks on the
+    matrix cores (32-bit products), the others token by token."""
+    _dev(x, b, c, dt, dt_bias, a_log, skip, state, entry_start, entry_first_pos, slots, out)
+    tokens = out.shape[0]
+    for t, what in ((x, "x"), (b, "b"), (c, "c"), (dt, "dt"), (state, "state"), (out, "out")):
+        _f32s(t, "state_space: " + what)
+    _need(x.shape == (tokens, heads * vdim) and b.shape == (tokens, groups * states) and c.shape == b.shape
+          and x.stride(1) == 1 and b.stride(1) == 1 and c.stride(1) == 1, "state_space: x, b and c")
+    _need(tokens == 1 or x.stride(0) == b.stride(0) == c.stride(0), "state_space: x, b and c need one row stride")
+    _need(heads % groups == 0, "state_space: heads must be a multiple of groups")
+    _need(dt.shape == (tokens, heads) and (dt.stride(1) == 1 or heads == 1), "state_space: dt")
+    _need(out.shape == (tokens, heads * vdim) and out.is_contiguous(), "state_space: out")
+    for t, what in ((dt_bias, "dt_bias"), (a_log, "a_log"), (skip, "skip")):
+        _f32(t, "state_space: " + what)
+        _need(t.numel() == heads, f"state_space: {what} is one number per head")
+    if states > STATE_SPACE_MAX_STATES:
+        raise UnsupportedError(f"state_space: {states} states are above the kernel's limit of {STATE_SPACE_MAX_STATES}")
+    _need(state.dim() == 2 and state.stride(1) == 1 and state.stride(0) % 4 == 0 and state.data_ptr() % 16 == 0
+          and state.shape[1] >= heads * state_space_head_floats(vdim, states), "state_space: state row")
+    _i32(entry_start, entry_first_pos, slots)
+    _entries_ok((entry_start, entry_first_pos, slots), num_entries)
+    _need(1 <= min_count <= max_count <= tokens, "state_space: token counts of the entries")
+    scores = None
+    if max_count > step_tokens:
+        scores = torch.empty((tokens, groups, STATE_SPACE_CHUNK), dtype=torch.float32, device=out.device)
+    fn = _fn("state_space", "vk_state_space", [_p, _p, _p, _ll, _p, _ll, _p, _p, _p, _p, _ll, _p, _p, _p, _i, _i, _i, _i, _i,
+                                               _p, _p, _i, _i, _i, _p])
+    _status(fn(_ptr(x), _ptr(b), _ptr(c), x.stride(0), _ptr(dt), dt.stride(0), _ptr(dt_bias), _ptr(a_log), _ptr(skip),
+               _ptr(state), state.stride(0), _ptr(entry_start), _ptr(entry_first_pos), _ptr(slots), num_entries, heads, groups,
+               vdim, states, _ptr(out), _ptr(scores), step_tokens, min_count, max_count, _stream()), "state_space")
+
+
+def gated_part_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, eps: float, parts: int, out: torch.Tensor) -> None:
+    """``v = y * silu(z)``, every one of ``parts`` equal parts of a row divided by its own root mean square, times
+    ``weight``; ``y`` 32-bit contiguous, ``z`` a 32-bit row-strided view."""
+    _dev(y, z, weight, out)
+    tokens, width = y.shape
+    _f32(y, "gated_part_norm: y")
+    _f32s(z, "gated_part_norm: z")
+    _need(z.shape == y.shape and z.stride(1) == 1 and out.shape == y.shape and out.is_contiguous() and width % parts == 0,
+          "gated_part_norm: shapes")
+    _need(weight.dtype == torch.float32 and weight.numel() == width and weight.is_contiguous(), "gated_part_norm: weight")
+    fn = _fn("state_space", "vk_gated_part_norm", [_p, _p, _ll, _p, _f, _i, _i, _i, _p, _i, _p])
+    _status(fn(_ptr(y), _ptr(z), z.stride(0), _ptr(weight), float(eps), parts, tokens, width, _ptr(out), _dt(out, "out"),
+               _stream()), "gated_part_norm")

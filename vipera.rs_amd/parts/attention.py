@@ -18,7 +18,9 @@ of the same token, and the blended values are what is cached; a ``"source"`` lay
 read it); ``qk_norm: "unit"`` (every q and k head divided by its root mean square *behind* the rotation, no weight);
 ``gate: "head_sigmoid"`` (one number per head, ``sigmoid(Wg h)_h``); ``sink`` (a learned logit per head that joins the
 softmax's denominator and nothing else); ``keep_first`` (with a window: the first that many positions of a sequence stay
-visible; the layer then keeps all its pages); ``rel_bias`` (``{"rows", "far"}``: a learned table ``[rows, heads]`` added
+visible; the layer then keeps all its pages); ``pairs: "interleaved"`` with ``rotary_dim`` (the rotation turns pairs
+``(2i, 2i + 1)`` of a head's first ``rotary_dim`` numbers: the rows of the q and k projections are reordered once, when they
+are loaded, so that the kernels' pairs are those); ``rel_bias`` (``{"rows", "far"}``: a learned table ``[rows, heads]`` added
 to the scaled score by the distance between query and key: one row per distance below ``rows / 2``, logarithmic steps
 from there to ``far``, the last row from ``far`` on); ``maps: 2`` with ``diff`` (differential attention: q and k hold two
 maps per head, each an attention of its own over the same values; the head's output is ``a_1 - lambda a_2`` with
@@ -42,6 +44,7 @@ from ..ops.attention import AttentionExtras, paged_attention
 from ..ops.linear import linear, linear_follow, split_qkv_plan, streams_in_wave_order
 from ..weights.checkpoint import MATRIX, VECTOR, TensorSpec
 from .base import KVCacheSpec, Mixer, register_mixer
+from .rotary import pairs_apart
 
 
 def _cat(tensors: List[torch.Tensor]) -> torch.Tensor:
@@ -124,7 +127,7 @@ class Attention(Mixer):
         # the kernel that rotates and norms in one pass, in 32-bit from the product's sums
         if (self.qk_norm == "unit" or self.maps > 1) and self.value_mix:
             raise UnsupportedError("attention: value_mix beside qk_norm \"unit\" or several maps is not implemented")
-        self.prepares = (self.qk_norm in ("unit", "head") or self.maps > 1) and not self.value_mix
+        self.prepares = self.qk_norm != "whole" and not self.value_mix
         self.extras = AttentionExtras(keep_first=self.keep_first)
         self.subtract = 0.0
         scale = p.get("scale")
@@ -177,6 +180,10 @@ class Attention(Mixer):
         base = f"{self.prefix}{self.spec.params['name']}."
         names = _tensor_names(self.spec.params)
         parts = [tensors[base + names[n]] for n in "qkv"]
+        if self.spec.params.get("pairs") == "interleaved":
+            rotary_dim = int(self.spec.params["rotary_dim"])
+            parts[0] = pairs_apart(parts[0], self.heads * self.maps, self.head_dim, 0, rotary_dim)
+            parts[1] = pairs_apart(parts[1], self.kv_heads * self.maps, self.head_dim, 0, rotary_dim)
         if self.gate:
             parts.append(tensors[base + names["g"]])
         self.w_qkv = _cat(parts)
@@ -217,6 +224,10 @@ class Attention(Mixer):
     def check_supported(cls, spec: PartSpec, dtype: torch.dtype) -> None:
         p = spec.params
         heads, kv_heads, head_dim = int(p["heads"]) * int(p.get("maps") or 1), int(p["kv_heads"]), _padded_width(p)
+        if p.get("pairs") not in (None, "interleaved"):
+            raise UnsupportedError(f"attention: pairs {p.get('pairs')!r}; \"interleaved\" or none")
+        if p.get("pairs") and (p.get("qk_norm") in ("whole", "head") or p.get("qkv_bias")):
+            raise UnsupportedError("attention: interleaved pairs beside weights of q and k norms or biases are not implemented")
         if p.get("qk_norm") not in (None, "whole", "head", "unit"):
             raise UnsupportedError(f"attention: qk_norm {p.get('qk_norm')!r} is not implemented; \"whole\", \"head\", "
                                    "\"unit\" or none")
@@ -298,7 +309,7 @@ class Attention(Mixer):
             written = () if reads_only else (cache.k, cache.v, batch.entry_of_token, batch.block_tables[cache.group])
             kernels.head_prepare(proj, self.q_norm, self.k_norm, bool(self.qk_norm), self.qk_norm != "unit", eps,
                                  batch.positions, inv_freq, rotary_dim, self.heads, self.kv_heads, self.maps,
-                                 self.head_dim, self.value_dim, width, qkv, *written)
+                                 self.head_dim, self.value_dim, width, qkv, *written, amplitude=position.amplitude)
         elif self.qk_norm == "whole" and first is None:
             kernels.whole_norm_pack(proj, self.q_norm, self.k_norm, eps, self.heads, self.kv_heads, self.head_dim,
                                     self.value_dim, width, qkv)
@@ -322,6 +333,9 @@ class Attention(Mixer):
         attn = self.runtime.empty((tokens, heads * width))
         paged_attention(qkv, cache.k, cache.v, attn, batch, table, heads, self.kv_heads, width, self.scale,
                         self.mask, self.softcap, self.extras)
+        if self.maps == 1 and not self.gate and width == self.value_dim:      # nothing to unpack
+            linear(attn, self.w_o, self.b_o, residual, accumulate=accumulate)
+            return
         values = self.runtime.empty((tokens, self.heads * self.value_dim))
         gate = proj[:, self.q_width + self.kv_width + self.kv_heads * self.value_dim:] if self.gate else None
         if self.maps > 1 or self.gate == "head_sigmoid":

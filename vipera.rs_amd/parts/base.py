@@ -120,6 +120,10 @@ class Norm(Part):
         """``(self.forward(x), other.forward(x))``: two norms of the same rows; a kind that can runs them as one launch."""
         return self.forward(x), other.forward(x)
 
+    def as_kernel(self):
+        """``(kind, weight, bias, eps)`` as ``kernels.streams_step`` applies a norm, or None for a norm it does not know."""
+        return None
+
     def handoff(self, tokens: int) -> Optional[NormHandoff]:
         """A :class:`NormHandoff` for ``tokens`` rows if this norm can be split between its neighbours, else None."""
         return None
@@ -132,6 +136,9 @@ class Norm(Part):
 
 
 class PositionEncoding(Part):
+    #: what the rotation's sines and cosines are multiplied by
+    amplitude = 1.0
+
     def fused_rotary(self):
         return None
 

@@ -16,6 +16,7 @@ from ..ops.linear import linear
 from ..errors import InvalidArgumentError
 from ..weights.checkpoint import MATRIX, VECTOR, TensorSpec
 from .base import FeedForward, Part, part_class, register_embedding, register_ffn, register_head
+from .streams import ResidualStreams
 
 
 def _tensor_name(spec: PartSpec, prefix: str) -> str:
@@ -30,7 +31,8 @@ class Embedding(Part):
     """``params``: ``vocab``, ``width``, ``name`` / ``tensor``, ``norm`` (a norm right after the table), ``scale`` (the
     rows are multiplied by it), ``side`` (``{"tensor": name, "width": columns}``: a second table with a row per token id,
     whose rows for the step's tokens are gathered once a step and left in ``batch.shared`` for the layers that read
-    their own columns of it, see :class:`TokenSide`)."""
+    their own columns of it, see :class:`TokenSide`), ``streams`` (the layers keep that many residual streams, all equal
+    to these rows at the start: ``embed`` returns :class:`~vipera_rs_amd.parts.streams.ResidualStreams`)."""
 
     reads_device_tokens = True  # forward() takes (source, sampled): ids may be read from the device
 
@@ -45,6 +47,7 @@ class Embedding(Part):
         self.norm = part_class("norm", norm.kind)(norm, prefix, runtime) if norm is not None else None
         scale = spec.params.get("scale")
         self.scale = float(scale) if scale is not None else 1.0
+        self.streams = int(spec.params.get("streams") or 0)
         self.side = spec.params.get("side")
         self.side_table: Optional[torch.Tensor] = None
 
@@ -81,16 +84,15 @@ class Embedding(Part):
             rows = self.runtime.empty((batch.num_tokens, self.side_table.shape[1]), torch.float32)
             kernels.embed_gather(self.side_table, batch.tokens, rows, *device_ids)
             batch.shared[SIDE_ROWS] = rows
-        return self.forward(batch.tokens, batch.num_tokens, *device_ids)
+        rows = self.forward(batch.tokens, batch.num_tokens, *device_ids)
+        return ResidualStreams(rows, self.streams) if self.streams else rows
 
     def forward(self, tokens: torch.Tensor, count: int, source: Optional[torch.Tensor] = None,
                 sampled: Optional[torch.Tensor] = None) -> torch.Tensor:
         """Rows of the table for ``tokens``; where ``source`` is not negative the id is read from
         ``sampled`` on the device instead (see ``kernels.embed_gather``)."""
         out = self.runtime.empty((count, self.width), torch.float32)
-        kernels.embed_gather(self.table, tokens, out, source, sampled)
-        if self.scale != 1.0:
-            kernels.scale_(out, self.scale)
+        kernels.embed_gather(self.table, tokens, out, source, sampled, self.scale)
         if self.norm is not None:
             out = self.norm.forward(out, out=self.runtime.empty((count, self.width), torch.float32))
         return out

@@ -1,4 +1,5 @@
-"""Norms.  RMSNorm: ``out = (x * rsqrt(mean(x^2) + eps)) * weight`` with the sum in 32-bit; Dynamic Tanh below.
+"""Norms.  RMSNorm: ``out = (x * rsqrt(mean(x^2) + eps)) * weight`` with the sum in 32-bit; layer norm and Dynamic Tanh
+below.
 With ``one_plus`` the stored weight lies around zero and the gain is ``1 + weight`` (added once, in 32-bit, when the
 weight is loaded).  ``add_into`` is the norm behind a sublayer: the normed rows are added to the 32-bit residual.
 
@@ -12,6 +13,7 @@ from typing import Dict, List, Optional
 import torch
 
 from ..config.base import PartSpec
+from ..errors import UnsupportedError
 from ..ops import kernels
 from ..weights.checkpoint import VECTOR, TensorSpec
 from .base import Norm, NormHandoff, register_norm
@@ -62,6 +64,9 @@ class RMSNorm(Norm):
         kernels.rmsnorm_add(y, self.weight, self.eps, residual)
         return follow.forward(residual) if follow is not None else None
 
+    def as_kernel(self):
+        return "rms", self.weight, None, self.eps
+
     def handoff(self, tokens: int) -> Optional[NormHandoff]:
         if self.runtime.dtype != torch.bfloat16 or self.weight is None or self.weight.dtype != torch.float32:
             return None
@@ -74,6 +79,52 @@ class RMSNorm(Norm):
         if out is None:
             out = self.runtime.empty((count, self.width))
         kernels.rmsnorm(x, self.weight, self.eps, out, rows)
+        return out
+
+
+class LayerNorm(Norm):
+    """Layer norm: ``out = (x - mean) / sqrt(mean((x - mean)^2) + eps) * weight + bias``, all in 32-bit.  ``params``:
+    ``width``, ``eps``, ``tensor`` (the weight's name after the part's prefix; the bias is ``<tensor>.b``)."""
+
+    def __init__(self, spec: PartSpec, prefix: str, runtime):
+        super().__init__(spec, prefix, runtime)
+        self.width, self.eps = int(spec.params["width"]), float(spec.params["eps"])
+        self.weight = self.bias = None
+
+    @classmethod
+    def declare(cls, spec: PartSpec, prefix: str) -> List[TensorSpec]:
+        name, width = f"{prefix}{spec.params['tensor']}", int(spec.params["width"])
+        return [TensorSpec(name, (width,), VECTOR, "one_plus_normal"), TensorSpec(name + ".b", (width,), VECTOR)]
+
+    @classmethod
+    def check_supported(cls, spec: PartSpec, dtype: torch.dtype) -> None:
+        if int(spec.params["width"]) > kernels.STREAMS_MAX_WIDTH:
+            raise UnsupportedError(f"layer norm: a width of {spec.params['width']} is above the kernel's limit of "
+                                   f"{kernels.STREAMS_MAX_WIDTH}")
+
+    def load(self, tensors: Dict[str, torch.Tensor]) -> None:
+        name = f"{self.prefix}{self.spec.params['tensor']}"
+        self.weight, self.bias = tensors[name], tensors[name + ".b"]
+
+    def as_kernel(self):
+        return "layer", self.weight, self.bias, self.eps
+
+    def forward(self, x, out=None, rows=None):
+        count = x.shape[0] if rows is None else rows.numel()
+        if out is None:
+            out = self.runtime.empty((count, self.width))
+        kernels.streams_step(x, 1, None, None, None, None, None, out, *self.as_kernel(), rows=rows)
+        return out
+
+    def add_into(self, y: torch.Tensor, residual: torch.Tensor, follow=None, as_input: bool = False):
+        normed = self.forward(y, out=torch.empty_like(y))
+        kernels.axpby(normed, 1.0, normed, 0.0, residual, accumulate=True)
+        if follow is not None:
+            return follow.forward(residual)
+        if not as_input or self.runtime.dtype == torch.float32:
+            return residual if as_input else None
+        out = self.runtime.empty(tuple(residual.shape))
+        kernels.activation(residual, "none", out)            # a change of type
         return out
 
 
@@ -115,4 +166,5 @@ class DynamicTanh(Norm):
 
 
 register_norm("rmsnorm", RMSNorm)
+register_norm("layernorm", LayerNorm)
 register_norm("dyt", DynamicTanh)

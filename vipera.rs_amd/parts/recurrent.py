@@ -33,6 +33,12 @@ silu; ``W_x x = [dt | B | C]``; ``step = softplus(W_dt dt + dt_bias)``; per chan
 ``S[c, n] <- exp(step_c A[c, n]) S[c, n] + step_c x_c B_n`` with ``A = -exp(A_log)``; ``y_c = S[c, :] . C + D_c x_c``;
 ``y * silu(z)`` goes through ``Wo``.
 
+``state_space``: Mamba-2 (Dao and Gu, "Transformers are SSMs: Generalized Models and Efficient Algorithms Through Structured
+State Space Duality").  ``W_in h = [z | x | B | C | dt]`` (``heads * vdim``, ``heads * vdim``, ``groups * state``, ``groups *
+state``, ``heads`` rows); x, B and C pass a short causal convolution per channel with a bias, and silu; ``step = softplus(dt +
+dt_bias)``; per head ``S <- exp(-exp(A_log) step) S + step B x^T`` (``state x vdim``; the heads of a group share B and C),
+``y = S^T C + D x``; ``y * silu(z)`` is RMS-normed in ``norm_groups`` equal parts, times ``norm``, and goes through ``Wo``.
+
 All keep their state in 32-bit in the request's slot: the matrices, and what the next token needs of this one (the
 convolution's last inputs; the last ``h``).  An entry that starts at position 0 starts from zeros.  Everything the
 kernels look at lies on the device, so a step of single tokens can be captured.
@@ -526,7 +532,96 @@ class SelectiveScan(Mixer):
         linear(y, self.w_o, None, residual, accumulate=accumulate)
 
 
+class StateSpace(Mixer):
+    """``params``: ``hidden``, ``heads``, ``vdim``, ``state`` (numbers per channel), ``groups`` (of heads that share B and C),
+    ``norm_groups``, ``conv`` (taps), ``eps``, ``name``; tensors ``<name>.in | conv | conv.b | dt_bias | A_log | D | norm | o``.
+
+    A portion of a prompt runs in chunks on the matrix cores (32-bit products), an entry of a few tokens token by token;
+    see ``kernels.state_space``."""
+
+    can_overwrite = True
+
+    def __init__(self, spec: PartSpec, prefix: str, runtime):
+        super().__init__(spec, prefix, runtime)
+        p = spec.params
+        self.hidden, self.heads, self.vdim = int(p["hidden"]), int(p["heads"]), int(p["vdim"])
+        self.states, self.groups, self.norm_groups = int(p["state"]), int(p["groups"]), int(p["norm_groups"])
+        self.taps, self.eps = int(p["conv"]), float(p["eps"])
+        self.inner, self.channels, self.rows = self._sizes(p)
+        self.w_in = self.conv = self.conv_b = self.dt_bias = self.a_log = self.skip = self.norm = self.w_o = None
+
+    @staticmethod
+    def _sizes(p):
+        """Inner width, convolved channels, rows of the input product."""
+        inner = int(p["heads"]) * int(p["vdim"])
+        channels = inner + 2 * int(p["groups"]) * int(p["state"])
+        return inner, channels, inner + channels + int(p["heads"])
+
+    @classmethod
+    def declare(cls, spec: PartSpec, prefix: str) -> List[TensorSpec]:
+        p = spec.params
+        base = f"{prefix}{p['name']}."
+        heads, hidden = int(p["heads"]), int(p["hidden"])
+        inner, channels, rows = cls._sizes(p)
+        return [TensorSpec(base + "in", (rows, hidden), MATRIX),
+                TensorSpec(base + "conv", (channels, int(p["conv"])), VECTOR, std=0.5),
+                TensorSpec(base + "conv.b", (channels,), VECTOR),
+                TensorSpec(base + "dt_bias", (heads,), VECTOR, std=0.5), TensorSpec(base + "A_log", (heads,), VECTOR, std=0.5),
+                TensorSpec(base + "D", (heads,), VECTOR, std=0.5), TensorSpec(base + "norm", (inner,), VECTOR, "one_plus_normal"),
+                TensorSpec(base + "o", (hidden, inner), MATRIX)]
+
+    @classmethod
+    def _matrix_floats(cls, p) -> int:
+        return int(p["heads"]) * kernels.state_space_head_floats(int(p["vdim"]), int(p["state"]))
+
+    @classmethod
+    def declare_cache(cls, spec: PartSpec):
+        p = spec.params
+        floats = cls._matrix_floats(p) + (int(p["conv"]) - 1) * cls._sizes(p)[1]
+        return None, StateSpec(((floats + 3) // 4 * 4,), torch.float32)      # rows of whole 16-byte pieces
+
+    @classmethod
+    def check_supported(cls, spec: PartSpec, dtype: torch.dtype) -> None:
+        p = spec.params
+        if int(p["state"]) > kernels.STATE_SPACE_MAX_STATES:
+            raise UnsupportedError(f"state_space: {p['state']} states are above the kernel's limit of "
+                                   f"{kernels.STATE_SPACE_MAX_STATES}")
+        if int(p["conv"]) < 1:
+            raise UnsupportedError(f"state_space: the convolution needs at least one tap, got {p['conv']}")
+        if int(p["heads"]) % int(p["groups"]) or int(p["heads"]) * int(p["vdim"]) % int(p["norm_groups"]):
+            raise InvalidArgumentError(f"state_space: {p['heads']} heads of {p['vdim']} do not divide into {p['groups']} groups "
+                                       f"and {p['norm_groups']} parts of the norm")
+
+    def load(self, tensors: Dict[str, torch.Tensor]) -> None:
+        base = f"{self.prefix}{self.spec.params['name']}."
+        self.w_in, self.w_o = tensors[base + "in"], tensors[base + "o"]
+        self.conv, self.conv_b = tensors[base + "conv"], tensors[base + "conv.b"]
+        self.dt_bias, self.a_log, self.skip = tensors[base + "dt_bias"], tensors[base + "A_log"], tensors[base + "D"]
+        self.norm = tensors[base + "norm"]
+
+    def forward(self, h, batch, cache, state, position, residual, reads_only: bool = False, accumulate: bool = True) -> None:
+        tokens, entries = residual.shape[0], batch.num_entries
+        f32 = dict(dtype=torch.float32, device=residual.device)
+        proj = torch.empty((tokens, self.rows), **f32)              # 32-bit from the product's sums on
+        linear(h, self.w_in, None, proj)
+        z, dt = proj[:, :self.inner], proj[:, self.inner + self.channels:]
+        xbc = torch.empty((tokens, self.channels), **f32)
+        kernels.causal_conv(proj[:, self.inner:self.inner + self.channels], self.conv, self.conv_b, state,
+                            self._matrix_floats(self.spec.params), batch.entry_of_token, batch.entry_start,
+                            batch.entry_first_pos, batch.slots, xbc, None, entries)
+        b_col = self.inner
+        c_col = b_col + self.groups * self.states
+        y = torch.empty((tokens, self.inner), **f32)
+        kernels.state_space(xbc[:, :b_col], xbc[:, b_col:c_col], xbc[:, c_col:], dt, self.dt_bias, self.a_log, self.skip, state,
+                            batch.entry_start, batch.entry_first_pos, batch.slots, self.heads, self.groups, self.vdim,
+                            self.states, y, entries, min(batch.host_counts), batch.max_count)
+        gated = self.runtime.empty((tokens, self.inner))
+        kernels.gated_part_norm(y, z, self.norm, self.eps, self.norm_groups, gated)
+        linear(gated, self.w_o, None, residual, accumulate=accumulate)
+
+
 register_mixer("gated_delta", GatedDelta)
+register_mixer("state_space", StateSpace)
 register_mixer("matrix_memory", MatrixMemory)
 register_mixer("decay_attention", DecayAttention)
 register_mixer("selective_scan", SelectiveScan)
