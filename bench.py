@@ -92,7 +92,7 @@ def main() -> int:
                         help="also run one decode step (of --batch requests at --ctx) and one prefill eagerly with a "
                              "pair of GPU events around every kernel launch, and add the microseconds of each class of "
                              "kernel to the line (split_decode_us, split_prefill_us)")
-    parser.add_argument("--design", default="", choices=["", "gilidra", "zulesun", "muzasun", "lurirax"],
+    parser.add_argument("--design", default="", choices=["", "gilidra", "zulesun", "muzasun", "lurirax", "zeladra"],
                         help="instead of the headline measurement: prefill and decode of this design at layer sizes that "
                              "resemble a real model's (--size), beside the dense Qwen2 decoder of the same width, depth and "
                              "active feed-forward width, each with the time of every class of kernel")
@@ -460,6 +460,33 @@ def lurirax_shape(z):
             "embedding": {"scale": 1.0}, "layers": layers}
 
 
+def zeladra_shape(z):
+    """A Zeladra configuration of sizes ``z``: latent attention, the state-space recurrence (inner width twice the model's,
+    heads of 64, state 128, no feed-forward), attention in a window with kept first positions, a latent layer that reads
+    the first one's cache, the recurrence again, and so on; dense feed-forwards; four residual streams."""
+    heads = z["heads"]
+    dense = {"kind": "dense", "ff": z["top"] * z["ff"]}
+    latent = {"heads": heads, "dim": z["dim"], "rot_dim": z["rot"], "vdim": z["dim"], "q_rank": z["q_rank"],
+              "kv_rank": z["kv_rank"], "scale": (z["dim"] + z["rot"]) ** -0.5,
+              "rot": {"base": 1e6, "dims": z["rot"], "scaling": {"factor": 8.0, "fast": 32.0, "slow": 1.0, "original": 8192}}}
+    window = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": z["dim"], "vdim": z["dim"],
+              "mask": {"size": z["window"], "keep_first": 64}, "rot": {"base": 1e6, "dims": z["dim"] // 2},
+              "scale": z["dim"] ** -0.5}
+    space = {"heads": z["width"] // 32, "vdim": 64, "state": 128, "groups": 8, "norm_groups": 8, "conv": 4}
+    layers = []
+    for index in range(z["layers"]):
+        kind = index % 5
+        if kind in (0, 3):
+            mixer = dict(latent, kv_from=index - 3) if kind == 3 else dict(latent)
+            layers.append({"type": "latent_attention", "mixer": mixer, "mlp": dense})
+        elif kind == 2:
+            layers.append({"type": "attention", "mixer": window, "mlp": dense})
+        else:
+            layers.append({"type": "mamba2", "mixer": space, "mlp": None})
+    return {"architecture": "Zeladra", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-5}, "streams": 4,
+            "embedding": {"scale": 1.0}, "layers": layers}
+
+
 def dense_shape(z):
     """The dense Qwen2 decoder of the same width, depth, heads and active feed-forward width."""
     return dict(QWEN25_7B, num_hidden_layers=z["layers"], hidden_size=z["width"], num_attention_heads=z["heads"],
@@ -489,12 +516,15 @@ def design_comparison(args) -> int:
     gen = torch.Generator().manual_seed(0)
     out = {}
     # Gilidra beside the dense decoder; Zulesun and Muzasun each beside Gilidra, the engine's other decoder of
-    # recurrences and mixtures of experts behind Dynamic Tanh norms, and beside the dense decoder
+    # recurrences and mixtures of experts behind Dynamic Tanh norms, and beside the dense decoder; Zeladra beside Gilidra
+    # (latent attention) and Zulesun (a scan behind a convolution) and beside the dense decoder
     runs = ((("gilidra", gilidra_shape(z)), ("dense", dense_shape(z))) if args.design == "gilidra" else
             (("muzasun", muzasun_shape(z)), ("gilidra", gilidra_shape(z)), ("dense", dense_shape(z)))
             if args.design == "muzasun" else
             (("lurirax", lurirax_shape(z)), ("zulesun", zulesun_shape(z)), ("dense", dense_shape(z)))
             if args.design == "lurirax" else
+            (("zeladra", zeladra_shape(z)), ("gilidra", gilidra_shape(z)), ("zulesun", zulesun_shape(z)),
+             ("dense", dense_shape(z))) if args.design == "zeladra" else
             (("zulesun", zulesun_shape(z)), ("gilidra", gilidra_shape(z)), ("dense", dense_shape(z))))
     for name, shape in runs:
         config = config_from_dict(shape)
@@ -559,6 +589,7 @@ def design_comparison(args) -> int:
         torch.cuda.empty_cache()
     print(json.dumps({"metric": f"prefill and decode of {args.design} beside " + ("the dense decoder" if args.design == "gilidra"
                                                                                     else "Zulesun and the dense decoder" if args.design == "lurirax"
+                                                                                    else "Gilidra, Zulesun and the dense decoder" if args.design == "zeladra"
                                                                                     else "Gilidra and the dense decoder") + " of equal size",
                       "size": z, "dtype": args.dtype, "prefill_tokens": T, "ctx": ctx, "data": "synthetic: seeded random "
                       "weights and uniform-random token ids", **out}), flush=True)
