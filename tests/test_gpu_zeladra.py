@@ -245,7 +245,7 @@ def test_the_convolution_over_portions_and_single_tokens(channels, taps):
             kept = np.concatenate([np.zeros((taps - 1, channels)), past])[len(past):]
             state[slots[e], offset:] = dev(kept.reshape(-1))
     whole = [list(past) for past in histories]
-    for sizes in (counts, [1] * E, [3] + [1] * (E - 1), [1] * E):
+    for sizes in (counts, [1] * E, [3] + [1] * (E - 1), [1] * E, [5, 70, 1, 130, 16, 33, 2, 64], [2] * E):
         T = sum(sizes)
         starts = np.concatenate([[0], np.cumsum(sizes)])
         x = rng.standard_normal((T, channels + 5))

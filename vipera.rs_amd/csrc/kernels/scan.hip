@@ -256,6 +256,61 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const float* __restric
   if (yrun) yrun[(long long)t * C + c] = from_float<TO>(y);
 }
 
+// The same for up to four taps over longer portions: a thread takes CONV_TOKENS consecutive tokens of its channel and
+// keeps the last inputs in registers, so an input is read once (and the K - 1 before the first).  The sum's order is
+// causal_conv_kernel's.  Grid (ceil(tokens / CONV_TOKENS), ceil(C / 256)).
+constexpr int CONV_TOKENS = 16;
+template <int K, typename TO>
+__global__ __launch_bounds__(256) void causal_conv_run_kernel(const float* __restrict__ in, long long ldi,
+                                                              const float* __restrict__ conv,
+                                                              const float* __restrict__ bias, int C,
+                                                              const float* __restrict__ state, long long state_stride,
+                                                              long long conv_offset, const int* __restrict__ entry_of,
+                                                              const int* __restrict__ entry_start,
+                                                              const int* __restrict__ entry_first,
+                                                              const int* __restrict__ slots, int num_tokens,
+                                                              float* __restrict__ y32, TO* __restrict__ yrun) {
+  const int c = blockIdx.y * 256 + threadIdx.x;
+  if (c >= C) return;
+  const int t0 = blockIdx.x * CONV_TOKENS, t1 = min(t0 + CONV_TOKENS, num_tokens);
+  float weight[K], past[K - 1];
+#pragma unroll
+  for (int j = 0; j < K; ++j) weight[j] = conv[(long long)c * K + j];
+  const float b = bias ? bias[c] : 0.f;
+  // all inputs of the run are on their way before the first is used
+  float x[CONV_TOKENS];
+#pragma unroll
+  for (int i = 0; i < CONV_TOKENS; ++i) x[i] = in[(long long)min(t0 + i, num_tokens - 1) * ldi + c];
+  int of = -1;
+#pragma unroll
+  for (int i = 0; i < CONV_TOKENS; ++i) {
+    const int t = t0 + i;
+    if (t >= t1) break;
+    const int e = entry_of[t];
+    if (e != of) {                       // the run's first token, or another entry's
+      of = e;
+      const int offset = t - entry_start[e];
+      const bool fresh = entry_first[e] == 0;
+      const float* old = state + (long long)slots[e] * state_stride + conv_offset + c;
+#pragma unroll
+      for (int j = 0; j < K - 1; ++j) {
+        const int back = K - 1 - j;      // tokens before t
+        past[j] = back <= offset ? in[(long long)(t - back) * ldi + c] : fresh ? 0.f : old[(long long)(j + offset) * C];
+      }
+    }
+    float sum = b;
+#pragma unroll
+    for (int j = 0; j < K - 1; ++j) sum = fmaf(weight[j], past[j], sum);
+    sum = fmaf(weight[K - 1], x[i], sum);
+#pragma unroll
+    for (int j = 0; j + 1 < K - 1; ++j) past[j] = past[j + 1];
+    past[K - 2] = x[i];
+    const float y = scan_silu(sum);
+    y32[(long long)t * C + c] = y;
+    if (yrun) yrun[(long long)t * C + c] = from_float<TO>(y);
+  }
+}
+
 // The convolution's inputs of an entry's last taps - 1 tokens become the state; runs after the convolution has read
 // the old rows.  Grid (entries, ceil(C / 256)), a thread per channel.
 __global__ __launch_bounds__(256) void conv_keep_kernel(const float* __restrict__ in, long long ldi, int taps, int C,
@@ -336,14 +391,31 @@ extern "C" int vk_causal_conv(const float* in, long long ldi, const float* conv,
     VK_LAUNCH_CHECK();
     return 0;
   }
-  if (yrun == nullptr || run_dtype == DT_F32)
+  if (yrun != nullptr && run_dtype != DT_F32 && run_dtype != DT_BF16) return VK_BAD_ARGUMENT;
+  const bool wide = yrun == nullptr || run_dtype == DT_F32;
+  if (taps >= 2 && taps <= 4 && num_tokens >= 256) {
+    dim3 runs((num_tokens + CONV_TOKENS - 1) / CONV_TOKENS, grid.y);
+#define VK_CONV_RUN(K)                                                                                               \
+  if (wide)                                                                                                          \
+    causal_conv_run_kernel<K, float><<<runs, 256, 0, s>>>(in, ldi, conv, bias, C, state, state_stride, conv_offset,  \
+                                                          entry_of, entry_start, entry_first, slots, num_tokens, y32, \
+                                                          (float*)yrun);                                             \
+  else                                                                                                               \
+    causal_conv_run_kernel<K, bf16_t><<<runs, 256, 0, s>>>(in, ldi, conv, bias, C, state, state_stride, conv_offset, \
+                                                           entry_of, entry_start, entry_first, slots, num_tokens, y32, \
+                                                           (bf16_t*)yrun)
+    switch (taps) {
+      case 2: VK_CONV_RUN(2); break;
+      case 3: VK_CONV_RUN(3); break;
+      default: VK_CONV_RUN(4); break;
+    }
+#undef VK_CONV_RUN
+  } else if (wide)
     causal_conv_kernel<float><<<grid, 256, 0, s>>>(in, ldi, conv, bias, taps, C, state, state_stride, conv_offset,
                                                    entry_of, entry_start, entry_first, slots, y32, (float*)yrun);
-  else if (run_dtype == DT_BF16)
+  else
     causal_conv_kernel<bf16_t><<<grid, 256, 0, s>>>(in, ldi, conv, bias, taps, C, state, state_stride, conv_offset,
                                                     entry_of, entry_start, entry_first, slots, y32, (bf16_t*)yrun);
-  else
-    return VK_BAD_ARGUMENT;
   VK_LAUNCH_CHECK();
   if (taps > 1) {
     conv_keep_kernel<<<dim3(num_entries, grid.y), 256, 0, s>>>(in, ldi, taps, C, state, state_stride, conv_offset,

@@ -165,26 +165,164 @@ __global__ __launch_bounds__(256) void state_space_scores_kernel(StateSpace a, i
   }
 }
 
-// The chunks of one entry, in order, for one head and 16 of its channels.  Grid (tiles of P, heads, entries), four
-// waves: wave w gives the outputs of the chunk's tokens 16 w .. 16 w + 15 and keeps the state's tiles of 16 rows
-// w, w + 4, .. (TPW of them) in registers; LDS holds the whole state for the outputs.
+// The chunks of one entry, in order, for one head and 16 of its channels.  Grid (tiles of P, heads, entries), eight
+// waves: waves 0 to 3 give the outputs of the chunk's tokens 16 w .. 16 w + 15, waves 4 to 7 carry the state, each its
+// tiles of 16 state rows w, w + 4, .. (TPW of them) in registers.  LDS holds the state at the chunk's start, the
+// channels' inputs and what the decays give, each twice: while one chunk is worked on, the state waves leave the next
+// one's state and inputs and wave 0 its decays in the other half, so a chunk costs one barrier.  What a wave reads from
+// memory for the next chunk it asks for as soon as it has used this one's.
+//
+// Off the diagonal of the chunk's 16-token tiles exp(c_j - c_t) is taken as exp(c_j - c_e) exp(c_e - c_t) with e the last
+// token of j's tile: both factors are at most 1, the first is made once per token, the second once per lane and tile.
+struct ChunkDecays {
+  float c_hi[CHUNK], c_lo[CHUNK], step[CHUNK], from_start[CHUNK];
+  __attribute__((aligned(16))) float to_tile[CHUNK];   // dt_j exp(c_j - c_e)
+  __attribute__((aligned(16))) float to_end[CHUNK];    // dt_j exp(c_j - c_end)
+  float whole;                                         // exp(-c_end)
+};
+
+// One wave, a lane per token: step sizes and the running sums of the decays' exponents.
+__device__ __forceinline__ void chunk_decays(const StateSpace& a, int t0, int count, int last, int h, float rate, float bias,
+                                             ChunkDecays& d) {
+  const int lane = threadIdx.x & 63;
+  const float dt = lane < count ? ss_softplus(a.dt[(long long)min(t0 + lane, last - 1) * a.lddt + h] + bias) : 0.f;
+  double sum = (double)(rate * dt);
+#pragma unroll
+  for (int off = 1; off < WAVE; off <<= 1) {
+    const double before = __shfl_up(sum, off, WAVE);
+    if (lane >= off) sum += before;
+  }
+  const double end = __shfl(sum, WAVE - 1, WAVE), tile_end = __shfl(sum, lane | 15, WAVE);
+  const float hi = (float)sum;
+  d.c_hi[lane] = hi;
+  d.c_lo[lane] = (float)(sum - (double)hi);
+  d.step[lane] = dt;
+  d.from_start[lane] = expf(-hi);
+  d.to_tile[lane] = dt * expf((float)(sum - tile_end));
+  d.to_end[lane] = dt * expf((float)(sum - end));
+  if (lane == 0) d.whole = expf(-(float)end);
+}
+
 template <int TPW, bool VEC>
-__global__ __launch_bounds__(256) void state_space_chunk_kernel(StateSpace a, int min_tokens) {
+__global__ __launch_bounds__(512) void state_space_chunk_kernel(StateSpace a, int min_tokens) {
   constexpr int NT = 4 * TPW, NROW = 16 * NT + 4, TROW = CHUNK + 4;
-  __shared__ __attribute__((aligned(16))) float s_lds[16 * NROW];     // [channel][state]
-  __shared__ __attribute__((aligned(16))) float x_lds[16 * TROW];     // [channel][token]
-  __shared__ float c_hi[CHUNK], c_lo[CHUNK], step[CHUNK], from_start[CHUNK];
-  __shared__ __attribute__((aligned(16))) float to_end[CHUNK];
-  __shared__ float whole;                                             // the chunk's decay
+  __shared__ __attribute__((aligned(16))) float s_lds[2][16 * NROW];     // [channel][state]
+  __shared__ __attribute__((aligned(16))) float x_lds[2][16 * TROW];     // [channel][token]
+  __shared__ ChunkDecays decays[2];
   const int h = blockIdx.y, e = blockIdx.z, p0 = blockIdx.x * 16;
   const int first = a.entry_start[e], last = a.entry_start[e + 1];
   if (last - first < min_tokens || last <= first) return;
-  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, col = lane & 15, q = lane >> 4;
+  // (the wave's number in a scalar register: the two roles part by a scalar branch, so no wave meets the other's barriers)
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), w = wave & 3;
+  const int col = lane & 15, q = lane >> 4;
   const int P = a.P, N = a.N, Np = padded_states(N), g = h / (a.heads / a.groups);
-  const bool fresh = a.entry_first[e] == 0, live = p0 + col < P;
+  const bool live = p0 + col < P;
+  const float rate = expf(a.a_log[h]), bias = a.dt_bias[h];
+  if (wave < 4) {
+    // ---- outputs
+    const float skip = a.skip[h];
+    const float* cbase = a.c + (long long)g * N;
+    const float* mbase = a.scores + (long long)g * CHUNK + 4 * q;
+    f32x4 c[NT], m[4];
+    auto load_c = [&](int t0) {
+      const float* row = cbase + (long long)min(t0 + 16 * w + col, last - 1) * a.ld;
+#pragma unroll
+      for (int k = 0; k < NT; ++k) c[k] = load4<VEC>(row, 16 * k + 4 * q, N);
+    };
+    auto load_m = [&](int t0) {
+      const float* row = mbase + (long long)min(t0 + 16 * w + col, last - 1) * a.groups * CHUNK;
+#pragma unroll
+      for (int jt = 0; jt < 4; ++jt) m[jt] = jt <= w ? *(const f32x4*)(row + 16 * jt) : f32x4{0.f, 0.f, 0.f, 0.f};
+    };
+    load_c(first);
+    load_m(first);
+    if (w == 0) chunk_decays(a, first, min(CHUNK, last - first), last, h, rate, bias, decays[0]);
+    __syncthreads();
+    int half = 0;
+    for (int t0 = first; t0 < last; t0 += CHUNK, half ^= 1) {
+      const int count = min(CHUNK, last - t0);
+      const ChunkDecays& d = decays[half];
+      const float* s = s_lds[half] + col * NROW + 4 * q;
+      const float* x = x_lds[half] + col * TROW;
+      const int t_own = 16 * w + col;
+      const float t_hi = d.c_hi[t_own], t_lo = d.c_lo[t_own];
+      // what the state at the chunk's start gives
+      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int k = 0; k < NT; ++k) acc = mma4(c[k], *(const f32x4*)(s + 16 * k), acc);
+      const bool more = t0 + CHUNK < last;
+      if (more) load_c(t0 + CHUNK);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) acc[i] *= d.from_start[16 * w + 4 * q + i];
+      // the chunk's own tokens
+#pragma unroll
+      for (int jt = 0; jt < 4; ++jt) {
+        if (jt > w) continue;
+        const int j0 = 16 * jt + 4 * q;
+        f32x4 left;
+        if (jt < w) {
+          const float gone = (t_hi - d.c_hi[16 * jt + 15]) + (t_lo - d.c_lo[16 * jt + 15]);
+          const float rest = expf(-gone);
+          const f32x4 weight = *(const f32x4*)(d.to_tile + j0);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) left[i] = m[jt][i] * (weight[i] * rest);
+        } else {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int j = j0 + i;
+            const float gone = (t_hi - d.c_hi[j]) + (t_lo - d.c_lo[j]);
+            left[i] = j <= t_own ? m[jt][i] * (d.step[j] * expf(-gone)) : 0.f;
+          }
+        }
+        acc = mma4(left, *(const f32x4*)(x + j0), acc);
+      }
+      if (more) load_m(t0 + CHUNK);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = 16 * w + 4 * q + i;
+        if (t < count && live) a.y[((long long)(t0 + t) * a.heads + h) * P + p0 + col] = fmaf(skip, x[t], acc[i]);
+      }
+      if (more && w == 0)
+        chunk_decays(a, t0 + CHUNK, min(CHUNK, last - t0 - CHUNK), last, h, rate, bias, decays[half ^ 1]);
+      __syncthreads();
+    }
+    return;
+  }
+  // ---- the state
+  const bool fresh = a.entry_first[e] == 0;
   float* srow = a.state + (long long)a.slots[e] * a.state_stride + ((long long)h * P + min(p0 + col, P - 1)) * Np;
-  const float rate = expf(a.a_log[h]), bias = a.dt_bias[h], skip = a.skip[h];
-  f32x4 s[TPW];
+  const float* xbase = a.x + (long long)h * P + min(p0 + col, P - 1);
+  const int tid = threadIdx.x - 256, x_token = tid >> 4;       // channel col (= tid & 15) of tokens x_token + 16 i
+  f32x4 s[TPW], b[TPW][4];
+  float x_next[4];
+  auto load_x = [&](int t0) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) x_next[i] = xbase[(long long)min(t0 + x_token + 16 * i, last - 1) * a.ld];
+  };
+  auto keep_x = [&](int t0, float* dst) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      dst[col * TROW + x_token + 16 * i] = (t0 + x_token + 16 * i < last && live) ? x_next[i] : 0.f;
+  };
+  auto load_b = [&](int t0) {
+#pragma unroll
+    for (int k = 0; k < TPW; ++k) {
+      const int n = 16 * (w + 4 * k) + col;
+      const float* base = a.b + (long long)g * N + min(n, N - 1);
+      if (t0 + CHUNK <= last) {
+        const float* row = base + (long long)(t0 + 4 * q) * a.ld;
+#pragma unroll
+        for (int jt = 0; jt < 4; ++jt)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) b[k][jt][i] = row[(long long)(16 * jt + i) * a.ld];
+      } else {
+#pragma unroll
+        for (int jt = 0; jt < 4; ++jt)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) b[k][jt][i] = base[(long long)min(t0 + 16 * jt + 4 * q + i, last - 1) * a.ld];
+      }
+    }
+  };
 #pragma unroll
   for (int k = 0; k < TPW; ++k) {
     const int n = 16 * (w + 4 * k) + 4 * q;
@@ -193,103 +331,43 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(StateSpace a, in
 #pragma unroll
     for (int i = 0; i < 4; ++i)
       if (n + i >= N) s[k][i] = 0.f;
-    *(f32x4*)(s_lds + col * NROW + n) = s[k];
+    *(f32x4*)(s_lds[0] + col * NROW + n) = s[k];
   }
-  for (int t0 = first; t0 < last; t0 += CHUNK) {
-    const int count = min(CHUNK, last - t0);
-    // what comes from memory: C and the scores of this wave's tokens, B of this wave's state rows
-    const int mine = min(t0 + 16 * w + col, last - 1);
-    const float* crow = a.c + (long long)mine * a.ld + (long long)g * N;
-    f32x4 c[NT];
-#pragma unroll
-    for (int k = 0; k < NT; ++k) c[k] = load4<VEC>(crow, 16 * k + 4 * q, N);
-    const float* score = a.scores + ((long long)mine * a.groups + g) * CHUNK;
-    f32x4 m[4];
-#pragma unroll
-    for (int jt = 0; jt < 4; ++jt) m[jt] = jt <= w ? *(const f32x4*)(score + 16 * jt + 4 * q) : f32x4{0.f, 0.f, 0.f, 0.f};
-    f32x4 b[TPW][4];
-#pragma unroll
-    for (int k = 0; k < TPW; ++k) {
-      const int n = 16 * (w + 4 * k) + col;
-      const float* bcol = a.b + (long long)g * N + min(n, N - 1);
-#pragma unroll
-      for (int jt = 0; jt < 4; ++jt)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const float v = bcol[(long long)min(t0 + 16 * jt + 4 * q + i, last - 1) * a.ld];
-          b[k][jt][i] = n < N ? v : 0.f;
-        }
-    }
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int idx = threadIdx.x + 256 * i, t = idx >> 4, p = idx & 15;
-      const float v = a.x[(long long)min(t0 + t, last - 1) * a.ld + (long long)h * P + min(p0 + p, P - 1)];
-      x_lds[p * TROW + t] = (t < count && p0 + p < P) ? v : 0.f;
-    }
-    if (w == 0) {        // a lane per token: step sizes and the sums of the decays' exponents
-      const float dt = lane < count ? ss_softplus(a.dt[(long long)min(t0 + lane, last - 1) * a.lddt + h] + bias) : 0.f;
-      double sum = (double)(rate * dt);
-#pragma unroll
-      for (int off = 1; off < WAVE; off <<= 1) {
-        const double before = __shfl_up(sum, off, WAVE);
-        if (lane >= off) sum += before;
-      }
-      const double end = __shfl(sum, WAVE - 1, WAVE);
-      const float hi = (float)sum;
-      c_hi[lane] = hi;
-      c_lo[lane] = (float)(sum - (double)hi);
-      step[lane] = dt;
-      from_start[lane] = expf(-hi);
-      to_end[lane] = dt * expf((float)(sum - end));
-      if (lane == 0) whole = expf(-(float)end);
-    }
-    __syncthreads();
-    // outputs: what the state at the chunk's start gives, then the chunk's own tokens
-    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int k = 0; k < NT; ++k) acc = mma4(c[k], *(const f32x4*)(s_lds + col * NROW + 16 * k + 4 * q), acc);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) acc[i] *= from_start[16 * w + 4 * q + i];
-    const int t_own = 16 * w + col;
-    const float t_hi = c_hi[t_own], t_lo = c_lo[t_own];
-#pragma unroll
-    for (int jt = 0; jt < 4; ++jt) {
-      if (jt > w) continue;
-      const int j0 = 16 * jt + 4 * q;
-      f32x4 left;
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int j = j0 + i;
-        const float gone = (t_hi - c_hi[j]) + (t_lo - c_lo[j]);
-        left[i] = j <= t_own ? m[jt][i] * (step[j] * expf(-gone)) : 0.f;
-      }
-      acc = mma4(left, *(const f32x4*)(x_lds + col * TROW + j0), acc);
-    }
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int t = 16 * w + 4 * q + i;
-      if (t < count && live)
-        a.y[((long long)(t0 + t) * a.heads + h) * P + p0 + col] = fmaf(skip, x_lds[col * TROW + t], acc[i]);
-    }
-    // the state at the chunk's end
+  load_x(first);
+  load_b(first);
+  keep_x(first, x_lds[0]);
+  __syncthreads();
+  int half = 0;
+  for (int t0 = first; t0 < last; t0 += CHUNK, half ^= 1) {
+    const bool more = t0 + CHUNK < last;
+    if (more) load_x(t0 + CHUNK);
+    const ChunkDecays& d = decays[half];
+    const float* x = x_lds[half] + col * TROW + 4 * q;
     f32x4 right[4];
 #pragma unroll
     for (int jt = 0; jt < 4; ++jt) {
-      const f32x4 x = *(const f32x4*)(x_lds + col * TROW + 16 * jt + 4 * q), weight = *(const f32x4*)(to_end + 16 * jt + 4 * q);
+      const f32x4 v = *(const f32x4*)(x + 16 * jt), weight = *(const f32x4*)(d.to_end + 16 * jt + 4 * q);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) right[jt][i] = x[i] * weight[i];
+      for (int i = 0; i < 4; ++i) right[jt][i] = v[i] * weight[i];
     }
-    const float keep = whole;
+    const float keep = d.whole;
 #pragma unroll
     for (int k = 0; k < TPW; ++k) {
+      const int n = 16 * (w + 4 * k);
 #pragma unroll
       for (int i = 0; i < 4; ++i) s[k][i] *= keep;
 #pragma unroll
       for (int jt = 0; jt < 4; ++jt) s[k] = mma4(b[k][jt], right[jt], s[k]);
-    }
-    __syncthreads();     // everyone has read this chunk's LDS
 #pragma unroll
-    for (int k = 0; k < TPW; ++k) *(f32x4*)(s_lds + col * NROW + 16 * (w + 4 * k) + 4 * q) = s[k];
+      for (int i = 0; i < 4; ++i)
+        if (n + 4 * q + i >= N) s[k][i] = 0.f;      // rows past N: B of the last row stood in for them
+      *(f32x4*)(s_lds[half ^ 1] + col * NROW + n + 4 * q) = s[k];
+    }
+    if (more) {
+      load_b(t0 + CHUNK);
+      keep_x(t0 + CHUNK, x_lds[half ^ 1]);
+    }
+    __syncthreads();
   }
   if (live) {
 #pragma unroll
@@ -302,41 +380,74 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(StateSpace a, in
 
 // ---------------------------------------------------------------------------------------------
 // v = y * silu(z); every one of `parts` equal parts of a row over its own root mean square; times the weight.
-// Grid (tokens, parts); a part of up to 16 numbers a thread stays in registers.
-template <typename TO>
+// Grid (ceil(tokens / tokens a workgroup), parts): a part is taken by blockDim.x threads, V consecutive numbers each
+// in KEPT places, which stay in registers across the sum; where one wave is enough for a part a workgroup takes four tokens.
+template <int V, int KEPT, typename TO>
 __global__ __launch_bounds__(256) void gated_part_norm_kernel(const float* __restrict__ y, const float* __restrict__ z,
                                                               long long ldz, const float* __restrict__ weight, float eps,
-                                                              int width, int part, TO* __restrict__ out) {
+                                                              int width, int part, int num_tokens, TO* __restrict__ out) {
   __shared__ float scratch[16];
-  const long long t = blockIdx.x;
+  typedef float vec __attribute__((ext_vector_type(V)));
+  typedef TO outvec __attribute__((ext_vector_type(V)));
+  const long long t = (long long)blockIdx.x * blockDim.y + threadIdx.y;
+  if (t >= num_tokens) return;          // only whole waves: with several tokens a workgroup there is no barrier
   const int at = blockIdx.y * part;
   const float* ys = y + t * width + at;
   const float* zs = z + t * ldz + at;
-  TO* dst = out + t * width + at;
-  constexpr int KEPT = 16;
-  float v[KEPT], sum = 0.f;
-  const bool kept = part <= KEPT * (int)blockDim.x;
+  vec v[KEPT];
+  float sum = 0.f;
 #pragma unroll
   for (int i = 0; i < KEPT; ++i) {
-    const int c = threadIdx.x + blockDim.x * i;
-    v[i] = c < part ? ys[c] * ss_silu(zs[c]) : 0.f;
-    sum = fmaf(v[i], v[i], sum);
-  }
-  if (!kept)
-    for (int c = threadIdx.x + blockDim.x * KEPT; c < part; c += blockDim.x) {
-      const float u = ys[c] * ss_silu(zs[c]);
-      sum = fmaf(u, u, sum);
+    const int c = (threadIdx.x + blockDim.x * i) * V;
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[i][j] = 0.f;
+    if (c < part) {
+      const vec a = *(const vec*)(ys + c), b = *(const vec*)(zs + c);
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        v[i][j] = a[j] * ss_silu(b[j]);
+        sum = fmaf(v[i][j], v[i][j], sum);
+      }
     }
-  sum = block_sum(sum, scratch);
+  }
+  sum = blockDim.y > 1 ? wave_sum(sum) : block_sum(sum, scratch);
   const float inv = 1.0f / sqrtf(sum / (float)part + eps);
+  TO* dst = out + t * width + at;
 #pragma unroll
   for (int i = 0; i < KEPT; ++i) {
-    const int c = threadIdx.x + blockDim.x * i;
-    if (c < part) dst[c] = from_float<TO>(v[i] * inv * weight[at + c]);
+    const int c = (threadIdx.x + blockDim.x * i) * V;
+    if (c < part) {
+      const vec w = *(const vec*)(weight + at + c);
+      outvec o;
+#pragma unroll
+      for (int j = 0; j < V; ++j) o[j] = from_float<TO>(v[i][j] * inv * w[j]);
+      *(outvec*)(dst + c) = o;
+    }
   }
-  if (!kept)
-    for (int c = threadIdx.x + blockDim.x * KEPT; c < part; c += blockDim.x)
-      dst[c] = from_float<TO>(ys[c] * ss_silu(zs[c]) * inv * weight[at + c]);
+}
+
+template <typename TO>
+int launch_part_norm(const float* y, const float* z, long long ldz, const float* weight, float eps, int width, int part,
+                     int parts, int num_tokens, bool vector, TO* out, hipStream_t s) {
+  const int units = vector ? part / 4 : part;
+  const bool one_wave = units <= 128 && num_tokens >= 64;       // a few tokens spread over more workgroups instead
+  const dim3 block = one_wave ? dim3(64, 4) : dim3(units >= 256 ? 256 : (units + 63) / 64 * 64);
+  const int kept = (units + (int)block.x - 1) / (int)block.x;
+  const dim3 grid((num_tokens + block.y - 1) / block.y, parts);
+#define VK_PART(V, KEPT) \
+  gated_part_norm_kernel<V, KEPT, TO><<<grid, block, 0, s>>>(y, z, ldz, weight, eps, width, part, num_tokens, out)
+  if (vector) {
+    if (kept <= 2) VK_PART(4, 2);
+    else if (kept <= 16) VK_PART(4, 16);
+    else return VK_UNSUPPORTED_SIZE;
+  } else {
+    if (kept <= 4) VK_PART(1, 4);
+    else if (kept <= 64) VK_PART(1, 64);
+    else return VK_UNSUPPORTED_SIZE;
+  }
+#undef VK_PART
+  VK_LAUNCH_CHECK();
+  return 0;
 }
 }  // namespace
 
@@ -381,8 +492,8 @@ extern "C" int vk_state_space(const float* x, const float* b, const float* c, lo
     dim3 grid((P + 15) / 16, heads, num_entries);
     const int tiles = ((N + 15) / 16 + 3) / 4;
 #define VK_CHUNK(TPW)                                                                   \
-  if (vec) state_space_chunk_kernel<TPW, true><<<grid, 256, 0, s>>>(a, limit + 1);      \
-  else state_space_chunk_kernel<TPW, false><<<grid, 256, 0, s>>>(a, limit + 1)
+  if (vec) state_space_chunk_kernel<TPW, true><<<grid, 512, 0, s>>>(a, limit + 1);      \
+  else state_space_chunk_kernel<TPW, false><<<grid, 512, 0, s>>>(a, limit + 1)
     switch (tiles) {
       case 1: VK_CHUNK(1); break;
       case 2: VK_CHUNK(2); break;
@@ -400,15 +511,11 @@ extern "C" int vk_gated_part_norm(const float* y, const float* z, long long ldz,
   if (num_tokens <= 0) return 0;
   if (width < 1 || parts < 1 || width % parts || parts > 65535) return VK_BAD_ARGUMENT;
   const int part = width / parts;
-  const int threads = part >= 1024 ? 256 : part >= 512 ? 128 : 64;
-  dim3 grid(num_tokens, parts);
+  const bool vector = part % 4 == 0 && ldz % 4 == 0 && (((uintptr_t)y | (uintptr_t)z | (uintptr_t)weight | (uintptr_t)out) & 15) == 0;
   hipStream_t s = (hipStream_t)stream;
   if (out_dtype == DT_F32)
-    gated_part_norm_kernel<float><<<grid, threads, 0, s>>>(y, z, ldz, weight, eps, width, part, (float*)out);
-  else if (out_dtype == DT_BF16)
-    gated_part_norm_kernel<bf16_t><<<grid, threads, 0, s>>>(y, z, ldz, weight, eps, width, part, (bf16_t*)out);
-  else
-    return VK_BAD_ARGUMENT;
-  VK_LAUNCH_CHECK();
-  return 0;
+    return launch_part_norm<float>(y, z, ldz, weight, eps, width, part, parts, num_tokens, vector, (float*)out, s);
+  if (out_dtype == DT_BF16)
+    return launch_part_norm<bf16_t>(y, z, ldz, weight, eps, width, part, parts, num_tokens, vector, (bf16_t*)out, s);
+  return VK_BAD_ARGUMENT;
 }
