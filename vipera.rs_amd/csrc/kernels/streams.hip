@@ -74,20 +74,36 @@ __global__ __launch_bounds__(256) void streams_step_kernel(StreamsStep a, TO* __
 #pragma unroll
     for (int q = 0; q < N; ++q) mix[s][q] = (in && q < S && a.y) ? a.mix[s * S + q] : 0.f;
   }
+  // Up to EARLY places: everything the row needs is asked for at once, the norm's weights too, ahead of the first use
+  // (a step of few tokens is all latency).  A place past the row's end asks for the last columns and drops them.
+  constexpr bool EARLY = KEPT <= 4;
+  constexpr int XS = EARLY ? KEPT : 1;
+  Cols<V> x[XS][N], y[XS], weight[XS], bias[XS];
+  auto ask = [&](int i, int at) {
+    const int c = min(((int)threadIdx.x + (int)blockDim.x * i) * V, W - V);
+#pragma unroll
+    for (int s = 0; s < N; ++s)
+      if (s < S) x[at][s] = cols_load<V>(src + s * a.stream_stride + c);
+    if (a.y) y[at] = cols_load<V>(a.y + t * W + c);
+    if constexpr (EARLY) {
+      if (a.weight) weight[at] = cols_load<V>(a.weight + c);
+      if (a.bias) bias[at] = cols_load<V>(a.bias + c);
+    }
+  };
+  if constexpr (EARLY) {
+#pragma unroll
+    for (int i = 0; i < KEPT; ++i) ask(i, i);
+  }
   Cols<V> u[KEPT];
   float sum = 0.f;
 #pragma unroll
   for (int i = 0; i < KEPT; ++i) {
-    const int c = ((int)threadIdx.x + (int)blockDim.x * i) * V;
+    const int c = ((int)threadIdx.x + (int)blockDim.x * i) * V, at = EARLY ? i : 0;
 #pragma unroll
     for (int j = 0; j < V; ++j) u[i].v[j] = 0.f;
     if (c >= W) continue;
-    Cols<V> x[N];
-#pragma unroll
-    for (int s = 0; s < N; ++s)
-      if (s < S) x[s] = cols_load<V>(src + s * a.stream_stride + c);
+    if constexpr (!EARLY) ask(i, 0);
     if (a.y) {
-      const Cols<V> y = cols_load<V>(a.y + t * W + c);
       Cols<V> n[N];
 #pragma unroll
       for (int q = 0; q < N; ++q) {
@@ -97,22 +113,22 @@ __global__ __launch_bounds__(256) void streams_step_kernel(StreamsStep a, TO* __
           float v = 0.f;
 #pragma unroll
           for (int s = 0; s < N; ++s)
-            if (s < S) v = fmaf(mix[s][q], x[s].v[j], v);
-          n[q].v[j] = fmaf(share[q], y.v[j], v);
+            if (s < S) v = fmaf(mix[s][q], x[at][s].v[j], v);
+          n[q].v[j] = fmaf(share[q], y[at].v[j], v);
         }
       }
 #pragma unroll
       for (int q = 0; q < N; ++q)
         if (q < S) {
-          x[q] = n[q];
-          if (a.dst) cols_store<V>(a.dst + (t * S + q) * W + c, x[q]);
+          x[at][q] = n[q];
+          if (a.dst) cols_store<V>(a.dst + (t * S + q) * W + c, n[q]);
         }
     }
 #pragma unroll
     for (int s = 0; s < N; ++s)
       if (s < S) {
 #pragma unroll
-        for (int j = 0; j < V; ++j) u[i].v[j] = fmaf(read[s], x[s].v[j], u[i].v[j]);
+        for (int j = 0; j < V; ++j) u[i].v[j] = fmaf(read[s], x[at][s].v[j], u[i].v[j]);
       }
 #pragma unroll
     for (int j = 0; j < V; ++j) sum += a.norm == 1 ? u[i].v[j] * u[i].v[j] : u[i].v[j];
@@ -148,8 +164,8 @@ __global__ __launch_bounds__(256) void streams_step_kernel(StreamsStep a, TO* __
 #pragma unroll
     for (int j = 0; j < V; ++j) {
       o.v[j] = (u[i].v[j] - mean) * inv;
-      if (a.weight) o.v[j] *= a.weight[c + j];
-      if (a.bias) o.v[j] += a.bias[c + j];
+      if (a.weight) o.v[j] *= EARLY ? weight[EARLY ? i : 0].v[j] : a.weight[c + j];
+      if (a.bias) o.v[j] += EARLY ? bias[EARLY ? i : 0].v[j] : a.bias[c + j];
     }
     if constexpr (V == 4 && sizeof(TO) == 2) {
       typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
@@ -176,7 +192,8 @@ int launch_step(const StreamsStep& a, TO* out, int num_rows, bool vector, hipStr
     else if (kept <= 16) VK_STREAMS(4, 16);
     else return VK_UNSUPPORTED_SIZE;
   } else {
-    if (kept <= 8) VK_STREAMS(1, 8);
+    if (kept <= 4) VK_STREAMS(1, 4);
+    else if (kept <= 8) VK_STREAMS(1, 8);
     else if (kept <= 64) VK_STREAMS(1, 64);
     else return VK_UNSUPPORTED_SIZE;
   }
@@ -207,7 +224,7 @@ extern "C" int vk_streams_step(const float* src, long long token_stride, long lo
   if (streams > 8) return VK_UNSUPPORTED_SIZE;
   const StreamsStep a{src, token_stride, stream_stride, y, mix, share, dst, read, norm, weight, bias, eps, rows, streams, width};
   const bool vector = width % 4 == 0 && token_stride % 4 == 0 && stream_stride % 4 == 0 &&
-                      (((uintptr_t)src | (uintptr_t)y | (uintptr_t)dst | (uintptr_t)out) & 15) == 0;
+                      (((uintptr_t)src | (uintptr_t)y | (uintptr_t)dst | (uintptr_t)out | (uintptr_t)weight | (uintptr_t)bias) & 15) == 0;
   hipStream_t s = (hipStream_t)stream;
   if (out == nullptr || out_dtype == DT_F32) return launch_streams<float>(a, (float*)out, num_rows, vector, s);
   if (out_dtype == DT_BF16) return launch_streams<bf16_t>(a, (bf16_t*)out, num_rows, vector, s);
