@@ -965,9 +965,12 @@ __global__ __launch_bounds__(JOINED ? JOINED_WAVES * 64 : 64) __attribute__((amd
     early_pages = block_table[(size_t)entry * table_width + min(ps.page(chunk_index * chunk) + lane, table_width - 1)];
   const int pos = entry_first_pos[entry];
   const int lo = EXT ? first_visible(pos, window) : ((window > 0 && pos + 1 > window) ? pos + 1 - window : 0);
-  // a chunk that holds kept first positions starts with them; what lies between them and the window is masked
-  const int begin = (EXT && chunk_index * chunk < ex.keep_first) ? chunk_index * chunk : max(lo, chunk_index * chunk);
-  const int end = min(pos + 1, (chunk_index + 1) * chunk);
+  // a chunk that holds kept first positions starts with them; what lies between them and the window is masked, and where
+  // the window starts behind the chunk it ends with them
+  const bool keeps = EXT && chunk_index * chunk < ex.keep_first;
+  const int begin = keeps ? chunk_index * chunk : max(lo, chunk_index * chunk);
+  int end = min(pos + 1, (chunk_index + 1) * chunk);
+  if (keeps && lo >= end) end = min(end, ex.keep_first);
   const int head_in_group = hb * 16 + lr;
   const bool col_ok = head_in_group < group;
   const int h = kvh * group + head_in_group;
