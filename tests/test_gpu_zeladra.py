@@ -137,6 +137,44 @@ def test_a_layer_norm_of_a_large_mean_keeps_its_digits():
     assert rel_err(out.cpu().numpy(), P.layer_norm(np.float64(x), 1.0, 0.0, 1e-5)) < 2e-4
 
 
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_streams_and_layer_norms_beside_other_norms(dtype):
+    """The streams with a norm that their kernel applies itself (layer, RMS) and one that it does not know (Dynamic Tanh),
+    and a layer norm behind a sublayer, as another design may put them together."""
+    from vipera_rs_amd.config.base import PartSpec
+    from vipera_rs_amd.parts import part_class
+    from vipera_rs_amd.parts.streams import ResidualStreams
+    from vipera_rs_amd.runtime import Runtime
+
+    rng, runtime = np.random.default_rng(6), Runtime("cuda:0", dtype)
+    tokens, width, eps, tol = 5, 24, 1e-5, 1e-5 if dtype == "float32" else 1e-2
+    weight, bias, alpha = 1 + 0.2 * rng.standard_normal(width), 0.3 * rng.standard_normal(width), 0.7
+    row, y1, y2 = (rng.standard_normal((tokens, width)) for _ in range(3))
+    mix, share, read = rng.standard_normal((3, 3)), rng.standard_normal(3), rng.standard_normal(3)
+    two = np.repeat(row[None], 3, axis=0)
+    for y in (y1, y2):
+        two = np.einsum("st,skw->tkw", mix, two) + share[:, None, None] * y
+    u = np.einsum("s,skw->kw", read, two)
+    kinds = {"layernorm": lambda x: P.layer_norm(x, weight, bias, eps), "rmsnorm": lambda x: P.over_rms(x, eps) * weight,
+             "dyt": lambda x: np.tanh(alpha * x) * weight + bias}
+    for kind, apply in kinds.items():
+        norm = part_class("norm", kind)(PartSpec(kind, {"width": width, "eps": eps, "name": "n", "tensor": "n"}), "", runtime)
+        norm.load({"n": dev(weight), "n.b": dev(bias), "n.alpha": dev(np.array(alpha))})
+        x = ResidualStreams(dev(row), 3)
+        x.leave(dev(y1), dev(mix), dev(share))
+        x.leave(dev(y2), dev(mix), dev(share))           # nobody has read in between: the first joins now
+        rows = torch.tensor([3, 1], dtype=torch.int32, device="cuda")
+        assert rel_err(x.read_rows(norm, rows, runtime).float().cpu().numpy(), apply(two.sum(axis=0))[[3, 1]]) < tol, kind
+        assert rel_err(x.read(dev(read), norm, runtime).float().cpu().numpy(), apply(u)) < tol, kind
+        assert rel_err(x.total().cpu().numpy(), two.sum(axis=0)) < 1e-6 and x.pending is None
+        if kind == "layernorm":
+            stream = dev(row)
+            out = norm.add_into(dev(y1), stream, follow=norm)
+            assert rel_err(stream.cpu().numpy(), row + apply(y1)) < tol
+            assert rel_err(out.float().cpu().numpy(), apply(row + apply(y1))) < 2 * tol
+            assert rel_err(norm.add_into(dev(y2), stream, as_input=True).float().cpu().numpy(), row + apply(y1) + apply(y2)) < 2 * tol
+
+
 SPACES = [(1, 1, 4, 1), (4, 2, 12, 20), (6, 3, 10, 7), (2, 1, 64, 128), (8, 2, 40, 64), (3, 1, 16, 33), (2, 2, 24, 200), (4, 1, 20, 256)]
 
 
