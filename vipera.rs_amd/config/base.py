@@ -63,11 +63,14 @@ class ScheduleEntry:
     ``layer`` indexes the list of layer specs; a layer may appear more than
     once.  ``cache_of`` is ``None`` when the entry owns a cache (or state) of
     its own, else the index of the earlier schedule entry whose cache it reads
-    without writing.
+    without writing.  ``rejoins``: ahead of the entry the stream meets the
+    embedding's output again, through the part :meth:`ModelConfig.rejoin_spec`
+    names.
     """
 
     layer: int
     cache_of: Optional[int] = None
+    rejoins: bool = False
 
 
 class ModelConfig:
@@ -89,6 +92,10 @@ class ModelConfig:
 
     def embedding_spec(self) -> PartSpec:
         raise NotImplementedError
+
+    def rejoin_spec(self) -> Optional[PartSpec]:
+        """The part (of the rejoin family) that runs ahead of the run order's entries with ``rejoins``."""
+        return None
 
     def final_norm_spec(self) -> PartSpec:
         raise NotImplementedError

@@ -575,11 +575,13 @@ extern "C" int vk_scale(float* x, float factor, long long count, void* stream) {
 // One workgroup per row; the sum of squares in the order of `rmsnorm_kernel`'s general path.
 // With `next_out`: the new rows of the residual also leave as the input of what follows, in that part's type: normed
 // again (`next_weight`, `next_eps`: the norm in front of the next sublayer) or as they are (`next_weight` null).
+// `next_layer`: that norm is a layer norm, which takes the row's mean off first, with `next_bias` (or null).
 template <typename TO>
 __global__ __launch_bounds__(256) void rmsnorm_add_kernel(const float* __restrict__ y, const float* __restrict__ weight,
                                                           float* __restrict__ residual, int width, float eps,
-                                                          const float* __restrict__ next_weight, float next_eps,
-                                                          TO* __restrict__ next_out) {
+                                                          const float* __restrict__ next_weight,
+                                                          const float* __restrict__ next_bias, float next_eps,
+                                                          int next_layer, TO* __restrict__ next_out) {
   __shared__ float scratch[16];
   const float* src = y + (size_t)blockIdx.x * width;
   float* dst = residual + (size_t)blockIdx.x * width;
@@ -607,10 +609,19 @@ __global__ __launch_bounds__(256) void rmsnorm_add_kernel(const float* __restric
       const int c = threadIdx.x + 256 * i;
       x[i] = x[i] + v[i] * inv * w[i];
       if (c < width) dst[c] = x[i];
-      again += x[i] * x[i];
+      again += next_layer ? x[i] : x[i] * x[i];
     }
     if (out == nullptr) return;
     float next_inv = 1.0f;
+    if (next_weight && next_layer) {
+      const float mean = block_sum(again, scratch) / (float)width;
+      again = 0.f;
+#pragma unroll
+      for (int i = 0; i < KEPT; ++i) {
+        x[i] -= mean;
+        if ((int)threadIdx.x + 256 * i < width) again += x[i] * x[i];
+      }
+    }
     if (next_weight) {
       again = block_sum(again, scratch);
       next_inv = 1.0f / sqrtf(again / (float)width + next_eps);
@@ -618,7 +629,7 @@ __global__ __launch_bounds__(256) void rmsnorm_add_kernel(const float* __restric
 #pragma unroll
     for (int i = 0; i < KEPT; ++i) {
       const int c = threadIdx.x + 256 * i;
-      if (c < width) out[c] = from_float<TO>(next_weight ? x[i] * next_inv * nw[i] : x[i]);
+      if (c < width) out[c] = from_float<TO>(next_weight ? x[i] * next_inv * nw[i] + (next_bias ? next_bias[c] : 0.f) : x[i]);
     }
     return;
   }
@@ -633,29 +644,37 @@ __global__ __launch_bounds__(256) void rmsnorm_add_kernel(const float* __restric
   for (int i = threadIdx.x; i < width; i += 256) {
     const float x = dst[i] + src[i] * inv * weight[i];
     dst[i] = x;
-    again += x * x;
+    again += next_layer ? x : x * x;
   }
   if (out == nullptr) return;
   if (next_weight == nullptr) {
     for (int i = threadIdx.x; i < width; i += 256) out[i] = from_float<TO>(dst[i]);   // a thread reads what it wrote
     return;
   }
+  float mean = 0.f;
+  if (next_layer) {
+    mean = block_sum(again, scratch) / (float)width;
+    again = 0.f;
+    for (int i = threadIdx.x; i < width; i += 256) again += (dst[i] - mean) * (dst[i] - mean);
+  }
   again = block_sum(again, scratch);
   const float next_inv = 1.0f / sqrtf(again / (float)width + next_eps);
-  for (int i = threadIdx.x; i < width; i += 256) out[i] = from_float<TO>(dst[i] * next_inv * next_weight[i]);
+  for (int i = threadIdx.x; i < width; i += 256)
+    out[i] = from_float<TO>((dst[i] - mean) * next_inv * next_weight[i] + (next_bias ? next_bias[i] : 0.f));
 }
 
 extern "C" int vk_rmsnorm_add(const float* y, const float* weight, float* residual, int num_rows, int width, float eps,
-                              const float* next_weight, float next_eps, void* next_out, int next_dtype, void* stream) {
+                              const float* next_weight, const float* next_bias, float next_eps, int next_layer,
+                              void* next_out, int next_dtype, void* stream) {
   if (num_rows <= 0) return 0;
-  if (width <= 0) return VK_BAD_ARGUMENT;
+  if (width <= 0 || (next_bias && !next_layer)) return VK_BAD_ARGUMENT;
   hipStream_t s = (hipStream_t)stream;
   if (next_out == nullptr || next_dtype == DT_F32)
-    rmsnorm_add_kernel<float><<<num_rows, 256, 0, s>>>(y, weight, residual, width, eps, next_weight, next_eps,
-                                                       (float*)next_out);
+    rmsnorm_add_kernel<float><<<num_rows, 256, 0, s>>>(y, weight, residual, width, eps, next_weight, next_bias, next_eps,
+                                                       next_layer, (float*)next_out);
   else if (next_dtype == DT_BF16)
-    rmsnorm_add_kernel<bf16_t><<<num_rows, 256, 0, s>>>(y, weight, residual, width, eps, next_weight, next_eps,
-                                                        (bf16_t*)next_out);
+    rmsnorm_add_kernel<bf16_t><<<num_rows, 256, 0, s>>>(y, weight, residual, width, eps, next_weight, next_bias, next_eps,
+                                                        next_layer, (bf16_t*)next_out);
   else
     return VK_BAD_ARGUMENT;
   VK_LAUNCH_CHECK();
@@ -679,7 +698,7 @@ extern "C" int vk_axpby(const float* x, float a, const float* y, float b, float*
   return 0;
 }
 
-// out[r, c] = act(in[r, c]) (* mul[r, c]); rows of `in` and `mul` may be strided.
+// out[r, c] = act(in[r, c]) (* mul[r, c]); rows of all three may be strided.
 //   act 0: as it is (a change of type), 1: relu squared, 2: silu, 3: gelu (tanh form), 4: sigmoid
 __device__ __forceinline__ float apply_act(float z, int act) {
   switch (act) {
@@ -693,18 +712,18 @@ __device__ __forceinline__ float apply_act(float z, int act) {
 
 template <typename TI, typename TM, typename TO>
 __global__ void activation_kernel(const TI* __restrict__ in, long long ldi, const TM* __restrict__ mul, long long ldm,
-                                  TO* __restrict__ out, int width, long long total, int act) {
+                                  TO* __restrict__ out, long long ldo, int width, long long total, int act) {
   const long long idx = (long long)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= total) return;
   const long long r = idx / width;
   const int c = (int)(idx % width);
   float v = apply_act(to_float<TI>(in[r * ldi + c]), act);
   if (mul) v *= to_float<TM>(mul[r * ldm + c]);
-  out[idx] = from_float<TO>(v);
+  out[r * ldo + c] = from_float<TO>(v);
 }
 
 extern "C" int vk_activation(const void* in, int in_dtype, long long ldi, const void* mul, int mul_dtype, long long ldm,
-                             void* out, int out_dtype, int num_rows, int width, int act, void* stream) {
+                             void* out, int out_dtype, long long ldo, int num_rows, int width, int act, void* stream) {
   if (num_rows <= 0) return 0;
   if (width <= 0 || act < 0 || act > 4) return VK_BAD_ARGUMENT;
   const long long total = (long long)num_rows * width;
@@ -712,7 +731,7 @@ extern "C" int vk_activation(const void* in, int in_dtype, long long ldi, const 
   hipStream_t s = (hipStream_t)stream;
   if (mul == nullptr) mul_dtype = DT_F32;
 #define VK_ACT(TI, TM, TO)                                                                                          \
-  activation_kernel<TI, TM, TO><<<blocks, 256, 0, s>>>((const TI*)in, ldi, (const TM*)mul, ldm, (TO*)out, width, total, act)
+  activation_kernel<TI, TM, TO><<<blocks, 256, 0, s>>>((const TI*)in, ldi, (const TM*)mul, ldm, (TO*)out, ldo, width, total, act)
 #define VK_ACT_O(TI, TM)                                \
   if (out_dtype == DT_F32) VK_ACT(TI, TM, float);       \
   else if (out_dtype == DT_BF16) VK_ACT(TI, TM, bf16_t); \

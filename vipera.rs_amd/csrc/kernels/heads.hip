@@ -1,6 +1,7 @@
 // Work on the heads of an attention layer before and behind the paged attention kernels, and small per-row steps of
 // layers whose sublayers are normed behind instead of in front. All arithmetic is 32-bit.
 #include "common.h"
+#include "conv_state.h"
 
 namespace {
 constexpr int HEAD_REGS = 4;   // a lane keeps up to four numbers of a head: heads of up to 256 numbers
@@ -144,6 +145,259 @@ __global__ __launch_bounds__(256) void head_prepare_kernel(
 }
 
 // ---------------------------------------------------------------------------------------------
+// head_conv_prepare: the same for queries and keys that pass a short causal convolution over time first, and for values
+// that may be the (convolved) keys.
+//   proj [T, ldp]: q (heads * dim) | k (kv_heads * dim) | v (kv_heads * vdim, where the layer has values of its own)
+//   conv [(heads + kv_heads) * dim, taps], the last column is the current token's, or null (no convolution); it runs over q
+//              and k, ahead of norm and rotation. Inputs before an entry's first token come from the state row of its slot
+//              ((taps - 1) rows of (heads + kv_heads) * dim numbers, oldest first), or are zero for an entry at position 0.
+//              `keep`: every entry is one token, and the wave that reads a head's old inputs moves them on; otherwise
+//              conv_keep_kernel follows
+//   values     the keys as they leave the convolution, or v
+//   norm, rotation as in head_prepare with norm_first; `angles` [T, rot_dims / 2]: the step's (sine, cosine), amplitude
+//              included, or null: computed here
+//   q  [T, heads * W]; k_cache, v_cache as above: keys and values go into their pages and nowhere else
+// One wave per (run of TW tokens, head); it keeps the run's last inputs in registers, so that an input is read once (and
+// the taps - 1 before the first). K: the taps that stay in registers (fewer are padded with zeros in front), 0: any number,
+// read again for every token. A run's values leave as 16-byte pieces where they fill an aligned piece of a page.
+template <typename TO> struct ConvHeads {
+  const float* proj;
+  long long ldp;
+  const float* conv;
+  int taps;
+  float* state;
+  long long state_stride;
+  int keep;
+  const int *entry_of, *entry_start, *entry_first, *slots;
+  const float *q_weight, *k_weight;
+  int norm;
+  float eps;
+  const int* positions;
+  const float* inv_freq;
+  const float2* angles;
+  int rot_dims;
+  float amplitude;
+  int heads, kv_heads, dim, vdim, own_values, W, tokens;
+  TO *q, *k_cache, *v_cache;
+  const int* table;
+  int table_width, block_size;
+};
+
+template <typename TO, int R, int K, int TW>
+__global__ __launch_bounds__(256) void head_conv_prepare_kernel(ConvHeads<TO> a, long long units) {
+  __shared__ float turned[4][R * WAVE];
+  const int lane = threadIdx.x & (WAVE - 1), wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
+  const long long unit = (long long)blockIdx.x * (blockDim.x / WAVE) + wave;
+  if (unit >= units) return;                             // a wave's work is its own: no barrier follows
+  const int qk = a.heads + a.kv_heads, per_token = qk + (a.own_values ? a.kv_heads : 0);
+  const int u = (int)(unit % per_token);
+  const int t0 = (int)(unit / per_token) * TW, t1 = min(t0 + TW, a.tokens);
+  const bool is_q = u < a.heads, is_v = u >= qk;
+  const int g = is_q ? 0 : is_v ? u - qk : u - a.heads;
+  const int n = is_v ? a.vdim : a.dim;
+  const long long base = is_v ? (long long)qk * a.dim + (long long)g * a.vdim : (long long)u * a.dim;
+  const int C = qk * a.dim, taps = is_v || !a.conv ? 1 : a.taps;
+  const bool gives_values = is_v || (!is_q && !a.own_values);
+  constexpr int P = K > 1 ? K - 1 : 1;
+  float w[K > 0 ? K : 1][R], past[P][R], x[TW][R], norm_weight[R];
+  const float* weight = is_q ? a.q_weight : a.k_weight;
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int d = lane + WAVE * r;
+    const bool in = d < n;
+#pragma unroll
+    for (int i = 0; i < TW; ++i) x[i][r] = in ? a.proj[(long long)min(t0 + i, a.tokens - 1) * a.ldp + base + d] : 0.f;
+    if constexpr (K > 0) {
+#pragma unroll
+      for (int j = 0; j < K; ++j) {
+        const int at = j - (K - taps);                   // column of the stored taps
+        w[j][r] = !in || at < 0 ? 0.f : taps > 1 || (a.conv && !is_v) ? a.conv[(base + d) * taps + at] : 1.f;
+      }
+    }
+    norm_weight[r] = (in && a.norm && weight && !is_v) ? weight[d] : 1.f;
+  }
+  TO held[TW][R];
+  int of = -1, run_entry = -1, run_first = 0;
+#pragma unroll
+  for (int i = 0; i < TW; ++i) {
+    const int t = t0 + i;
+    if (t >= t1) break;
+    const int e = a.entry_of[t], pos = a.positions[t];
+    const int offset = t - a.entry_start[e];
+    const bool fresh = a.entry_first[e] == 0;
+    float* old = a.conv ? a.state + (long long)a.slots[e] * a.state_stride + base : nullptr;
+    // a channel's input `back` tokens before t; `back` is at least 1 and below taps
+    auto before = [&](int back, int d) -> float {
+      if (back <= offset) return a.proj[(long long)(t - back) * a.ldp + base + d];
+      return fresh ? 0.f : old[(long long)(taps - 1 - (back - offset)) * C + d];
+    };
+    float y[R];
+    if constexpr (K > 0) {
+      if (e != of) {                                     // the run's first token, or another entry's
+        of = e;
+#pragma unroll
+        for (int j = 0; j < K - 1; ++j)
+#pragma unroll
+          for (int r = 0; r < R; ++r) {
+            const int d = lane + WAVE * r, back = K - 1 - j;
+            past[j][r] = (d < n && back < taps) ? before(back, d) : 0.f;
+          }
+      }
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+        float sum = 0.f;
+#pragma unroll
+        for (int j = 0; j < K - 1; ++j) sum = fmaf(w[j][r], past[j][r], sum);
+        y[r] = fmaf(w[K - 1][r], x[i][r], sum);
+        if (TW == 1 && a.keep && taps > 1 && lane + WAVE * r < n) {
+          // row j of the state becomes the input taps - 2 - j tokens before this one
+#pragma unroll
+          for (int back = 0; back < K - 1; ++back)
+            if (back < taps - 1) old[(long long)(taps - 2 - back) * C + lane + WAVE * r] = back ? past[K - 1 - back][r] : x[i][r];
+        }
+#pragma unroll
+        for (int j = 0; j + 1 < K - 1; ++j) past[j][r] = past[j + 1][r];
+        past[P - 1][r] = x[i][r];
+      }
+    } else {
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+        const int d = lane + WAVE * r;
+        y[r] = 0.f;
+        if (d >= n) continue;
+        float sum = 0.f;
+        for (int j = 0; j + 1 < taps; ++j) {
+          const float v = before(taps - 1 - j, d);
+          sum = fmaf(a.conv[(base + d) * taps + j], v, sum);
+          if (TW == 1 && a.keep && j > 0) old[(long long)(j - 1) * C + d] = v;
+        }
+        y[r] = taps > 1 || (a.conv && !is_v) ? fmaf(a.conv[(base + d) * taps + taps - 1], x[i][r], sum) : x[i][r];
+        if (TW == 1 && a.keep && taps > 1) old[(long long)(taps - 2) * C + d] = x[i][r];
+      }
+    }
+    if (i == 0) {
+      run_entry = e;
+      run_first = pos;
+    } else if (e != run_entry) {
+      run_entry = -1;
+    }
+    const int page = is_q ? -1 : a.table[(size_t)e * a.table_width + pos / a.block_size], slot = pos % a.block_size;
+    if (gives_values) {
+#pragma unroll
+      for (int r = 0; r < R; ++r) held[i][r] = from_float<TO>(lane + WAVE * r < n ? y[r] : 0.f);
+    }
+    if (is_v) continue;
+    if (a.norm) {
+      float ss = 0.f;
+#pragma unroll
+      for (int r = 0; r < R; ++r) ss = fmaf(y[r], y[r], ss);
+      const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)n + a.eps);
+#pragma unroll
+      for (int r = 0; r < R; ++r) y[r] = y[r] * inv * norm_weight[r];
+    }
+    if (a.rot_dims > 0) {
+      const int half = a.rot_dims / 2;
+#pragma unroll
+      for (int r = 0; r < R; ++r) turned[wave][lane + WAVE * r] = y[r];
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+        const int d = lane + WAVE * r;
+        if (d >= a.rot_dims) continue;
+        const int pair = d < half ? d : d - half;
+        const float other = turned[wave][d < half ? d + half : d - half];
+        float sn, cs;
+        if (a.angles) {
+          const float2 v = a.angles[(long long)t * half + pair];
+          sn = v.x;
+          cs = v.y;
+        } else {
+          sincosf((float)pos * a.inv_freq[pair], &sn, &cs);
+          sn *= a.amplitude;
+          cs *= a.amplitude;
+        }
+        y[r] = d < half ? y[r] * cs - other * sn : y[r] * cs + other * sn;
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+    }
+    if (!is_q && page < 0) continue;
+    TO* dst = is_q ? a.q + ((long long)t * a.heads + u) * a.W
+                   : a.k_cache + (((size_t)page * a.kv_heads + g) * a.block_size + slot) * a.W;
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const int d = lane + WAVE * r;
+      if (d < a.W) dst[d] = from_float<TO>(d < n ? y[r] : 0.f);
+    }
+  }
+  if (!gives_values) return;
+  // the run's values, transposed: consecutive positions of a number lie side by side in its page
+  constexpr int PIECE = 16 / (int)sizeof(TO);
+  const bool whole = TW % PIECE == 0 && t1 - t0 == TW && run_entry >= 0 && run_first % TW == 0 && a.block_size % TW == 0;
+  if (whole) {
+    const int page = a.table[(size_t)run_entry * a.table_width + run_first / a.block_size], slot = run_first % a.block_size;
+    if (page < 0) return;
+    typedef TO piece_t __attribute__((ext_vector_type(PIECE)));
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const int d = lane + WAVE * r;
+      if (d >= a.W) continue;
+      TO* dst = a.v_cache + (((size_t)page * a.kv_heads + g) * a.W + d) * a.block_size + slot;
+#pragma unroll
+      for (int p = 0; p < TW / PIECE; ++p) {
+        piece_t v;
+#pragma unroll
+        for (int i = 0; i < PIECE; ++i) v[i] = held[(p * PIECE + i) % TW][r];
+        *(piece_t*)(dst + p * PIECE) = v;
+      }
+    }
+    return;
+  }
+#pragma unroll
+  for (int i = 0; i < TW; ++i) {
+    const int t = t0 + i;
+    if (t >= t1) break;
+    const int pos = a.positions[t];
+    const int page = a.table[(size_t)a.entry_of[t] * a.table_width + pos / a.block_size], slot = pos % a.block_size;
+    if (page < 0) continue;
+    TO* dst = a.v_cache + ((size_t)page * a.kv_heads + g) * a.W * a.block_size + slot;
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const int d = lane + WAVE * r;
+      if (d < a.W) dst[(size_t)d * a.block_size] = held[i][r];
+    }
+  }
+}
+
+template <typename TO> int launch_head_conv_prepare(const ConvHeads<TO>& a, hipStream_t s) {
+  const int per_token = a.heads + a.kv_heads * (a.own_values ? 2 : 1);
+  const bool runs = a.tokens >= 512;          // enough tokens that waves of eight of them still fill the GPU
+  const long long units = (long long)(runs ? (a.tokens + 7) / 8 : a.tokens) * per_token;
+  const long long blocks = (units + 3) / 4;
+  if (blocks > 0x7fffffffLL) return VK_UNSUPPORTED_SIZE;
+  const bool few_taps = !a.conv || a.taps <= 4, narrow = a.W <= 2 * WAVE;
+#define VK_HEADS(R, K, TW) head_conv_prepare_kernel<TO, R, K, TW><<<(unsigned)blocks, 256, 0, s>>>(a, units)
+#define VK_HEADS_K(R)                            \
+  if (few_taps) {                                \
+    if (runs) VK_HEADS(R, 4, 8);                 \
+    else VK_HEADS(R, 4, 1);                      \
+  } else {                                       \
+    if (runs) VK_HEADS(R, 0, 8);                 \
+    else VK_HEADS(R, 0, 1);                      \
+  }
+  if (narrow) {
+    VK_HEADS_K(2)
+  } else {
+    VK_HEADS_K(4)
+  }
+#undef VK_HEADS_K
+#undef VK_HEADS
+  VK_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---------------------------------------------------------------------------------------------
 // head_finish: the attention kernels' output, heads padded to W, becomes the output product's input.
 //   attn [T, heads * maps * W]
 //   maps 2: o = a_1 - lambda a_2 with the two maps of a head (differential attention); maps 1: o = a
@@ -260,6 +514,44 @@ extern "C" int vk_head_prepare(const float* proj, long long ldp, const float* q_
                                                                  entry_of_token, block_table, table_width, block_size);
   else
     return VK_BAD_ARGUMENT;
+  VK_LAUNCH_CHECK();
+  return 0;
+}
+
+extern "C" int vk_head_conv_prepare(const float* proj, long long ldp, const float* conv, int taps, float* state,
+                                    long long state_stride, const int* entry_of, const int* entry_start, const int* entry_first,
+                                    const int* slots, int num_entries, const float* q_weight, const float* k_weight, int norm,
+                                    float eps, const int* positions, const float* inv_freq, const float* angles, int rot_dims,
+                                    float amplitude, int num_tokens, int heads, int kv_heads, int dim, int vdim, int own_values,
+                                    int W, void* q, int dtype, void* k_cache, void* v_cache, const int* block_table,
+                                    int table_width, int block_size, void* stream) {
+  if (num_tokens <= 0) return 0;
+  if (heads < 1 || kv_heads < 1 || dim < 1 || vdim < 1 || W < dim || W < vdim || num_entries < 1 || taps < 1) return VK_BAD_ARGUMENT;
+  if (!proj || !q || !k_cache || !v_cache || !entry_of || !entry_start || !entry_first || !slots || !positions || !block_table ||
+      table_width <= 0 || block_size <= 0 || (!own_values && vdim != dim) || (conv && taps > 1 && !state))
+    return VK_BAD_ARGUMENT;
+  if (W > HEAD_REGS * WAVE) return VK_UNSUPPORTED_SIZE;
+  if (rot_dims < 0 || rot_dims > dim || (rot_dims & 1) || (rot_dims > 0 && !inv_freq && !angles)) return VK_BAD_ARGUMENT;
+  hipStream_t s = (hipStream_t)stream;
+  const int keep = num_tokens == num_entries;
+#define VK_CONV_HEADS(TO)                                                                                                      \
+  launch_head_conv_prepare<TO>(                                                                                                \
+      ConvHeads<TO>{proj, ldp, conv, conv ? taps : 1, state, state_stride, keep, entry_of, entry_start, entry_first, slots,    \
+                    q_weight, k_weight, norm, eps, positions, inv_freq, (const float2*)angles, rot_dims, amplitude, heads,     \
+                    kv_heads, dim, vdim, own_values, W, num_tokens, (TO*)q, (TO*)k_cache, (TO*)v_cache, block_table,           \
+                    table_width, block_size},                                                                                  \
+      s)
+  int status = VK_BAD_ARGUMENT;
+  if (dtype == DT_F32) status = VK_CONV_HEADS(float);
+  else if (dtype == DT_BF16) status = VK_CONV_HEADS(bf16_t);
+#undef VK_CONV_HEADS
+  if (status != 0 || !conv || taps == 1) return status;
+  // one token per entry and a wave per token: the state has moved on already (a run of eight tokens leaves it to this)
+  if (keep && num_tokens < 512) return 0;
+  const int channels = (heads + kv_heads) * dim;
+  dim3 rows(num_entries, (channels + 255) / 256);
+  if (rows.y > 65535) return VK_UNSUPPORTED_SIZE;
+  conv_keep_kernel<<<rows, 256, 0, s>>>(proj, ldp, taps, channels, state, state_stride, 0, entry_start, entry_first, slots);
   VK_LAUNCH_CHECK();
   return 0;
 }

@@ -160,19 +160,29 @@ __device__ __forceinline__ float expert_act(float g, float u, float limit, float
   return g * (1.0f / (1.0f + expf(-alpha * g))) * u;
 }
 
+// The activation of an expert without a gate: 1 the square of relu, 2 silu, 3 gelu (tanh form).
+__device__ __forceinline__ float plain_act(float z, int act) {
+  switch (act) {
+    case 1: { const float r = fmaxf(z, 0.f); return r * r; }
+    case 2: return z / (1.0f + expf(-z));
+    default: return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+  }
+}
+
 // Gate and up products of a tile with the experts' activation (expert_act above).
-// h: [T, width] (row of pair p is p / top); wg, wu: [E, ff, width]; act: [P places, ff].
-template <typename T>
+// h: [T, width] (row of pair p is p / top); wg, wu: [E, ff, width]; act: [P places, ff].  GATED false: experts without a
+// gate, plain_act of kind `plain` of the up product alone (wg is not read).
+template <typename T, bool GATED>
 __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ h, long long ldh,
                                                           const T* __restrict__ wg, const T* __restrict__ wu,
                                                           const int* __restrict__ offsets,
                                                           const int* __restrict__ order, const int* __restrict__ tiles,
                                                           const int* __restrict__ num_tiles, int top, int width, int ff,
-                                                          float limit, float alpha, const float* __restrict__ in_weights,
-                                                          T* __restrict__ act) {
+                                                          float limit, float alpha, int plain,
+                                                          const float* __restrict__ in_weights, T* __restrict__ act) {
   if ((int)blockIdx.x >= num_tiles[0]) return;
   __shared__ float As[16][MOE_TILE + 4];
-  __shared__ float Gs[16][MOE_TILE + 4];
+  __shared__ float Gs[GATED ? 16 : 1][MOE_TILE + 4];
   __shared__ float Us[16][MOE_TILE + 4];
   __shared__ int rows[MOE_TILE];
   const int e = tiles[2 * blockIdx.x], first = tiles[2 * blockIdx.x + 1];
@@ -189,7 +199,7 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ 
       const int r = i >> 4, kk = i & 15, k = k0 + kk, n = n0 + r;
       As[kk][r] = (rows[r] >= 0 && k < width) ? to_float<T>(h[(long long)rows[r] * ldh + k]) : 0.f;
       const bool in = n < ff && k < width;
-      Gs[kk][r] = in ? to_float<T>(g_w[(long long)n * width + k]) : 0.f;
+      if constexpr (GATED) Gs[kk][r] = in ? to_float<T>(g_w[(long long)n * width + k]) : 0.f;
       Us[kk][r] = in ? to_float<T>(u_w[(long long)n * width + k]) : 0.f;
     }
     __syncthreads();
@@ -200,14 +210,14 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ 
       for (int i = 0; i < 4; ++i) av[i] = As[kk][ty * 4 + i];
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        gv[j] = Gs[kk][tx * 4 + j];
+        if constexpr (GATED) gv[j] = Gs[kk][tx * 4 + j];
         uv[j] = Us[kk][tx * 4 + j];
       }
 #pragma unroll
       for (int i = 0; i < 4; ++i)
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-          ga[i][j] = fmaf(av[i], gv[j], ga[i][j]);
+          if constexpr (GATED) ga[i][j] = fmaf(av[i], gv[j], ga[i][j]);
           ua[i][j] = fmaf(av[i], uv[j], ua[i][j]);
         }
     }
@@ -222,7 +232,8 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ 
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
       if (n >= ff) continue;
-      act[(long long)(first + r) * ff + n] = from_float<T>(expert_act(w * ga[i][j], w * ua[i][j], limit, alpha));
+      act[(long long)(first + r) * ff + n] =
+          from_float<T>(GATED ? expert_act(w * ga[i][j], w * ua[i][j], limit, alpha) : plain_act(w * ua[i][j], plain));
     }
   }
 }
@@ -326,6 +337,43 @@ __global__ __launch_bounds__(256) void moe_gate_up_mma_kernel(const __bf16* __re
   }
 }
 
+// The up product of experts without a gate: a workgroup owns 128 columns of an expert's width.
+__global__ __launch_bounds__(256) void moe_up_mma_kernel(const __bf16* __restrict__ h, long long ldh,
+                                                         const __bf16* __restrict__ wu, const int* __restrict__ offsets,
+                                                         const int* __restrict__ order, const int* __restrict__ tiles,
+                                                         const int* __restrict__ num_tiles, int top, int width, int ff,
+                                                         int plain, const float* __restrict__ in_weights,
+                                                         __bf16* __restrict__ act) {
+  if ((int)blockIdx.x >= num_tiles[0]) return;
+  extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
+  __shared__ int rows[GT_TILE];
+  const int e = tiles[2 * blockIdx.x], first = tiles[2 * blockIdx.x + 1];
+  const int count = min(GT_TILE, offsets[e + 1] - first);
+  const int n0 = blockIdx.y * GT_TILE;
+  for (int i = threadIdx.x; i < GT_TILE; i += 256) rows[i] = i < count ? order[first + i] / top : -1;
+  __syncthreads();
+  const __bf16* u_w = wu + (long long)e * ff * width;
+  gt_f32x4 acc[4][4];
+  group_tile_mma([&](int r) -> const __bf16* { return rows[r] >= 0 ? h + (long long)rows[r] * ldh : nullptr; },
+                 [&](int r) -> const __bf16* { return n0 + r < ff ? u_w + (long long)(n0 + r) * width : nullptr; }, width, lds,
+                 acc);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, wm = wave >> 1, wn = wave & 1;
+  const int lr = lane & 15, lg = lane >> 4;
+#pragma unroll
+  for (int tm = 0; tm < 4; ++tm) {
+    const int r = wm * 64 + tm * 16 + lr;
+    if (r >= count) continue;
+    const float w = in_weights ? in_weights[order[first + r]] : 1.f;
+#pragma unroll
+    for (int tn = 0; tn < 4; ++tn)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int col = n0 + wn * 64 + tn * 16 + lg * 4 + i;
+        if (col < ff) act[(long long)(first + r) * ff + col] = (__bf16)plain_act(w * acc[tn][tm][i], plain);
+      }
+  }
+}
+
 __global__ __launch_bounds__(256) void moe_down_mma_kernel(const __bf16* __restrict__ act, const __bf16* __restrict__ wd,
                                                            const int* __restrict__ offsets,
                                                            const int* __restrict__ order,
@@ -359,16 +407,60 @@ __global__ __launch_bounds__(256) void moe_down_mma_kernel(const __bf16* __restr
   }
 }
 
-// residual[t, :] (+)= sum_j weights[t, j] * pair_out[t * top + j, :], j ascending (weights null: every weight is 1).
+// residual[t, :] (+)= sum_j weights[t, j] * pair_out[t * top + j, :], j ascending (weights null: every weight is 1), and
+// what joins a token's experts:
+struct Combine {
+  const float* extra;        // [T, width] 32-bit, or null: added too,
+  const float* extra_gate;   // times sigmoid(extra_gate[t * ldg]), or null: as it is
+  long long ldg;
+  bf16_t* stream;            // [T, width], or null: the residual's new rows in 16 bits
+};
+// A thread owns V consecutive columns of a row.
+template <int V>
 __global__ void moe_combine_kernel(const float* __restrict__ pair_out, const float* __restrict__ weights, int top,
-                                   int width, long long total, float* __restrict__ residual, int accumulate) {
-  const long long idx = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+                                   int width, long long total, float* __restrict__ residual, int accumulate, Combine with) {
+  typedef float fv __attribute__((ext_vector_type(V)));
+  typedef bf16_t bv __attribute__((ext_vector_type(V)));
+  const long long idx = ((long long)blockIdx.x * blockDim.x + threadIdx.x) * V;
   if (idx >= total) return;
   const long long t = idx / width;
   const int c = (int)(idx % width);
-  float sum = 0.f;
-  for (int j = 0; j < top; ++j) sum = fmaf(weights ? weights[t * top + j] : 1.f, pair_out[(t * top + j) * width + c], sum);
-  residual[idx] = accumulate ? residual[idx] + sum : sum;
+  fv sum = 0.f;
+  for (int j = 0; j < top; ++j) {
+    const float w = weights ? weights[t * top + j] : 1.f;
+    const fv v = *(const fv*)(pair_out + (t * top + j) * width + c);
+#pragma unroll
+    for (int i = 0; i < V; ++i) sum[i] = fmaf(w, v[i], sum[i]);
+  }
+  if (with.extra) {
+    const float g = with.extra_gate ? 1.0f / (1.0f + expf(-with.extra_gate[t * with.ldg])) : 1.f;
+    const fv v = *(const fv*)(with.extra + idx);
+#pragma unroll
+    for (int i = 0; i < V; ++i) sum[i] = fmaf(g, v[i], sum[i]);
+  }
+  if (accumulate) sum = *(const fv*)(residual + idx) + sum;
+  *(fv*)(residual + idx) = sum;
+  if (with.stream) {
+    bv b;
+#pragma unroll
+    for (int i = 0; i < V; ++i) b[i] = (bf16_t)sum[i];
+    *(bv*)(with.stream + idx) = b;
+  }
+}
+
+static int launch_combine(const float* pair_out, const float* weights, int num_tokens, int top, int width, float* residual,
+                          int accumulate, const Combine& with, hipStream_t s) {
+  const long long total = (long long)num_tokens * width;
+  const bool wide = width % 4 == 0 &&
+                    (((uintptr_t)pair_out | (uintptr_t)residual | (uintptr_t)with.extra) & 15) == 0 && ((uintptr_t)with.stream & 7) == 0;
+  if (wide)
+    moe_combine_kernel<4><<<(unsigned)((total / 4 + 255) / 256), 256, 0, s>>>(pair_out, weights, top, width, total, residual,
+                                                                              accumulate, with);
+  else
+    moe_combine_kernel<1><<<(unsigned)((total + 255) / 256), 256, 0, s>>>(pair_out, weights, top, width, total, residual,
+                                                                          accumulate, with);
+  VK_LAUNCH_CHECK();
+  return 0;
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -385,10 +477,9 @@ extern "C" int vk_moe_tile_rows(int dtype, int width, int ff, long long ldh) {
   return moe_on_matrix_cores(dtype, width, ff, ldh) ? GT_TILE : MOE_TILE;
 }
 
-extern "C" int vk_moe_route_steered(const float* logits, int experts, int top, int num_tokens, int tile_rows, int groups,
-                                    int keep, int all_scores, const float* correction, float weight_scale, long long ld,
-                                    int* ids, float* weights, int* offsets, int* order, int* tiles, int* num_tiles,
-                                    void* stream) {
+extern "C" int vk_moe_route(const float* logits, int experts, int top, int num_tokens, int tile_rows, int groups, int keep,
+                            int all_scores, const float* correction, float weight_scale, long long ld, int* ids,
+                            float* weights, int* offsets, int* order, int* tiles, int* num_tiles, void* stream) {
   if (tile_rows != MOE_TILE && tile_rows != GT_TILE) return VK_BAD_ARGUMENT;
   if (groups < 1 || keep < 1 || keep > groups || experts % groups != 0) return VK_BAD_ARGUMENT;
   if (groups > WAVE) return VK_UNSUPPORTED_SIZE;
@@ -414,98 +505,70 @@ extern "C" int vk_moe_route_steered(const float* logits, int experts, int top, i
   return 0;
 }
 
-extern "C" int vk_moe_route_grouped(const float* logits, int experts, int top, int num_tokens, int tile_rows, int groups,
-                                    int keep, int all_scores, int* ids, float* weights, int* offsets, int* order,
-                                    int* tiles, int* num_tiles, void* stream) {
-  if (all_scores > 2) return VK_BAD_ARGUMENT;
-  return vk_moe_route_steered(logits, experts, top, num_tokens, tile_rows, groups, keep, all_scores, nullptr, 1.f, 0, ids,
-                              weights, offsets, order, tiles, num_tiles, stream);
-}
-
-extern "C" int vk_moe_route(const float* logits, int experts, int top, int num_tokens, int tile_rows, int* ids,
-                            float* weights, int* offsets, int* order, int* tiles, int* num_tiles, void* stream) {
-  return vk_moe_route_grouped(logits, experts, top, num_tokens, tile_rows, 1, 1, 0, ids, weights, offsets, order, tiles,
-                              num_tiles, stream);
-}
-
 // accumulate 0: the weighted sums are written to `residual` instead of added to it.  weigh_input: a pair's weight
 // multiplies what its expert reads (w h, applied to the gate and up sums, which are linear in h) instead of what it
-// returns.
-extern "C" int vk_moe_experts_weighed(const void* h, long long ldh, const void* wg, const void* wu, const void* wd,
-                                      int dtype, const int* offsets, const int* order, const int* tiles,
-                                      const int* num_tiles, const float* weights, int num_tokens, int experts, int top,
-                                      int width, int ff, float limit, float alpha, void* act, float* pair_out,
-                                      float* residual, int accumulate, int weigh_input, void* stream) {
+// returns.  plain: 0 experts with a gate (limit, alpha), else experts without one and their activation (plain_act; wg is
+// not read).  extra, extra_gate, stream: see Combine.
+extern "C" int vk_moe_experts(const void* h, long long ldh, const void* wg, const void* wu, const void* wd, int dtype,
+                              const int* offsets, const int* order, const int* tiles, const int* num_tiles,
+                              const float* weights, int num_tokens, int experts, int top, int width, int ff, float limit,
+                              float alpha, int plain, void* act, float* pair_out, float* residual, int accumulate,
+                              int weigh_input, const float* extra, const float* extra_gate, long long ldg, void* stream_rows,
+                              void* stream) {
   if (num_tokens <= 0) return 0;
   const float* in_weights = weigh_input ? weights : nullptr;
   const float* out_weights = weigh_input ? nullptr : weights;
-  if (experts < 1 || top < 1 || width < 1 || ff < 1) return VK_BAD_ARGUMENT;
+  if (experts < 1 || top < 1 || width < 1 || ff < 1 || plain < 0 || plain > 3 || (!plain && !wg) || (extra_gate && !extra))
+    return VK_BAD_ARGUMENT;
   const int pairs = num_tokens * top;
   hipStream_t s = (hipStream_t)stream;
+  const Combine with{extra, extra_gate, ldg, (bf16_t*)stream_rows};
   if (moe_on_matrix_cores(dtype, width, ff, ldh)) {
     if (((uintptr_t)h | (uintptr_t)wg | (uintptr_t)wu | (uintptr_t)wd | (uintptr_t)act) & 15) return VK_BAD_ARGUMENT;
-    const int wide_tiles = vk_moe_max_tiles(pairs, experts, GT_TILE);
-    dim3 up(wide_tiles, (ff + 63) / 64), down(wide_tiles, (width + GT_TILE - 1) / GT_TILE);
+    const int wide_tiles = vk_moe_max_tiles(pairs, experts, GT_TILE), columns = plain ? GT_TILE : 64;
+    dim3 up(wide_tiles, (ff + columns - 1) / columns), down(wide_tiles, (width + GT_TILE - 1) / GT_TILE);
     if (up.y > 65535 || down.y > 65535) return VK_UNSUPPORTED_SIZE;
     static bool sized = false;
     if (!sized) {
-      hipError_t e1 = hipFuncSetAttribute((const void*)moe_gate_up_mma_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, GT_LDS_BYTES);
-      hipError_t e2 = hipFuncSetAttribute((const void*)moe_down_mma_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, GT_LDS_BYTES);
-      if (e1 != hipSuccess || e2 != hipSuccess) return (int)(e1 != hipSuccess ? e1 : e2);
+      for (const void* kernel : {(const void*)moe_gate_up_mma_kernel, (const void*)moe_up_mma_kernel, (const void*)moe_down_mma_kernel}) {
+        const hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, GT_LDS_BYTES);
+        if (e != hipSuccess) return (int)e;
+      }
       sized = true;
     }
-    moe_gate_up_mma_kernel<<<up, 256, GT_LDS_BYTES, s>>>((const __bf16*)h, ldh, (const __bf16*)wg, (const __bf16*)wu,
-                                                        offsets, order, tiles, num_tiles, top, width, ff, limit, alpha,
-                                                        in_weights, (__bf16*)act);
+    if (plain)
+      moe_up_mma_kernel<<<up, 256, GT_LDS_BYTES, s>>>((const __bf16*)h, ldh, (const __bf16*)wu, offsets, order, tiles, num_tiles,
+                                                     top, width, ff, plain, in_weights, (__bf16*)act);
+    else
+      moe_gate_up_mma_kernel<<<up, 256, GT_LDS_BYTES, s>>>((const __bf16*)h, ldh, (const __bf16*)wg, (const __bf16*)wu,
+                                                          offsets, order, tiles, num_tiles, top, width, ff, limit, alpha,
+                                                          in_weights, (__bf16*)act);
     VK_LAUNCH_CHECK();
     moe_down_mma_kernel<<<down, 256, GT_LDS_BYTES, s>>>((const __bf16*)act, (const __bf16*)wd, offsets, order, tiles,
                                                         num_tiles, width, ff, pair_out);
     VK_LAUNCH_CHECK();
-    const long long all = (long long)num_tokens * width;
-    moe_combine_kernel<<<(unsigned)((all + 255) / 256), 256, 0, s>>>(pair_out, out_weights, top, width, all, residual, accumulate);
-    VK_LAUNCH_CHECK();
-    return 0;
+    return launch_combine(pair_out, out_weights, num_tokens, top, width, residual, accumulate, with, s);
   }
   const int max_tiles = vk_moe_max_tiles(pairs, experts, MOE_TILE);
   dim3 up_grid(max_tiles, (ff + MOE_TILE - 1) / MOE_TILE), down_grid(max_tiles, (width + MOE_TILE - 1) / MOE_TILE);
   if (up_grid.y > 65535 || down_grid.y > 65535) return VK_UNSUPPORTED_SIZE;
+#define VK_MOE_UP(T, GATED)                                                                                            \
+  moe_gate_up_kernel<T, GATED><<<up_grid, 256, 0, s>>>((const T*)h, ldh, (const T*)wg, (const T*)wu, offsets, order, tiles, \
+                                                       num_tiles, top, width, ff, limit, alpha, plain, in_weights, (T*)act)
+#define VK_MOE_PRODUCTS(T)                                                                                             \
+  if (plain) VK_MOE_UP(T, false);                                                                                      \
+  else VK_MOE_UP(T, true);                                                                                             \
+  VK_LAUNCH_CHECK();                                                                                                   \
+  moe_down_kernel<T><<<down_grid, 256, 0, s>>>((const T*)act, (const T*)wd, offsets, order, tiles, num_tiles, width, ff, pair_out)
   if (dtype == DT_F32) {
-    moe_gate_up_kernel<float><<<up_grid, 256, 0, s>>>((const float*)h, ldh, (const float*)wg, (const float*)wu,
-                                                      offsets, order, tiles, num_tiles, top, width, ff, limit, alpha,
-                                                      in_weights, (float*)act);
-    VK_LAUNCH_CHECK();
-    moe_down_kernel<float><<<down_grid, 256, 0, s>>>((const float*)act, (const float*)wd, offsets, order, tiles,
-                                                     num_tiles, width, ff, pair_out);
+    VK_MOE_PRODUCTS(float);
   } else if (dtype == DT_BF16) {
-    moe_gate_up_kernel<bf16_t><<<up_grid, 256, 0, s>>>((const bf16_t*)h, ldh, (const bf16_t*)wg, (const bf16_t*)wu,
-                                                       offsets, order, tiles, num_tiles, top, width, ff, limit, alpha,
-                                                       in_weights, (bf16_t*)act);
-    VK_LAUNCH_CHECK();
-    moe_down_kernel<bf16_t><<<down_grid, 256, 0, s>>>((const bf16_t*)act, (const bf16_t*)wd, offsets, order, tiles,
-                                                      num_tiles, width, ff, pair_out);
+    VK_MOE_PRODUCTS(bf16_t);
   } else {
     return VK_BAD_ARGUMENT;
   }
+#undef VK_MOE_PRODUCTS
+#undef VK_MOE_UP
   VK_LAUNCH_CHECK();
-  const long long total = (long long)num_tokens * width;
-  moe_combine_kernel<<<(unsigned)((total + 255) / 256), 256, 0, s>>>(pair_out, out_weights, top, width, total, residual, accumulate);
-  VK_LAUNCH_CHECK();
-  return 0;
-}
-
-extern "C" int vk_moe_experts_into(const void* h, long long ldh, const void* wg, const void* wu, const void* wd, int dtype,
-                                   const int* offsets, const int* order, const int* tiles, const int* num_tiles,
-                                   const float* weights, int num_tokens, int experts, int top, int width, int ff,
-                                   float limit, float alpha, void* act, float* pair_out, float* residual,
-                                   int accumulate, void* stream) {
-  return vk_moe_experts_weighed(h, ldh, wg, wu, wd, dtype, offsets, order, tiles, num_tiles, weights, num_tokens, experts,
-                                top, width, ff, limit, alpha, act, pair_out, residual, accumulate, 0, stream);
-}
-
-extern "C" int vk_moe_experts(const void* h, long long ldh, const void* wg, const void* wu, const void* wd, int dtype,
-                              const int* offsets, const int* order, const int* tiles, const int* num_tiles,
-                              const float* weights, int num_tokens, int experts, int top, int width, int ff,
-                              float limit, float alpha, void* act, float* pair_out, float* residual, void* stream) {
-  return vk_moe_experts_into(h, ldh, wg, wu, wd, dtype, offsets, order, tiles, num_tiles, weights, num_tokens, experts,
-                             top, width, ff, limit, alpha, act, pair_out, residual, 1, stream);
+  return launch_combine(pair_out, out_weights, num_tokens, top, width, residual, accumulate, with, s);
 }

@@ -17,7 +17,7 @@ import torch
 
 from ..config.base import ModelConfig, ScheduleEntry
 from ..errors import InvalidArgumentError
-from ..parts.base import KVCacheSpec, StateSpec, part_class
+from ..parts.base import FollowingNorm, KVCacheSpec, StateSpec, part_class
 from ..weights.checkpoint import TensorSpec
 
 
@@ -50,6 +50,9 @@ def declare_model(config: ModelConfig) -> List[TensorSpec]:
     specs += part_class("embedding", emb.kind).declare(emb, "")
     for layer in config.layer_specs():
         specs += part_class("block", layer.block).declare(layer)
+    rejoin = config.rejoin_spec()
+    if rejoin is not None:
+        specs += part_class("rejoin", rejoin.kind).declare(rejoin, "")
     norm = config.final_norm_spec()
     specs += part_class("norm", norm.kind).declare(norm, "")
     head = config.head_spec()
@@ -69,6 +72,9 @@ def check_model(config: ModelConfig, dtype) -> None:
     part_class("embedding", emb.kind).check_supported(emb, dtype)
     for layer in config.layer_specs():
         part_class("block", layer.block).check_supported(layer, dtype)
+    rejoin = config.rejoin_spec()
+    if rejoin is not None:
+        part_class("rejoin", rejoin.kind).check_supported(rejoin, dtype)
     norm = config.final_norm_spec()
     part_class("norm", norm.kind).check_supported(norm, dtype)
     head = config.head_spec()
@@ -98,8 +104,12 @@ class DecoderModel:
         self.layers = [part_class("block", spec.block)(spec, runtime) for spec in config.layer_specs()]
         self.final_norm = part_class("norm", norm.kind)(norm, "", runtime)
         self.head = part_class("head", head.kind)(head, "", runtime)
+        rejoin = config.rejoin_spec()
+        self.rejoin = part_class("rejoin", rejoin.kind)(rejoin, "", runtime) if rejoin is not None else None
         self.schedule = list(config.schedule())
         check_schedule(self.schedule, len(self.layers))
+        if self.rejoin is None and any(entry.rejoins for entry in self.schedule):
+            raise InvalidArgumentError("the run order has entries that rejoin the embedding's output, but no part that does it")
         self.vocab_size = self.head.vocab
         self.loaded = False
 
@@ -110,6 +120,8 @@ class DecoderModel:
         self.embedding.load(tensors)
         for layer in self.layers:
             layer.load(tensors)
+        if self.rejoin is not None:
+            self.rejoin.load(tensors)
         self.final_norm.load(tensors)
         self.head.load(tensors)
         self.loaded = True
@@ -135,7 +147,11 @@ class DecoderModel:
         x = self.embedding.embed(batch)
         tokens = x.shape[0]
         incoming = None
+        if self.rejoin is not None:
+            self.rejoin.keep(x, batch)
         for index, entry in enumerate(self.schedule):
+            if entry.rejoins:
+                self.rejoin.forward(x, batch)
             owner = index if entry.cache_of is None else entry.cache_of
             layer = self.layers[entry.layer]
             if not layer.hands_off:
@@ -144,10 +160,12 @@ class DecoderModel:
                 continue
             # the next layer's first norm may be prepared by this layer's last product (see parts.NormHandoff)
             outgoing = None
-            if index + 1 < len(self.schedule) and layer.fills_outgoing():
+            if index + 1 < len(self.schedule) and not self.schedule[index + 1].rejoins:
                 following = self.layers[self.schedule[index + 1].layer]
-                if following.hands_off:
+                if following.hands_off and layer.fills_outgoing():
                     outgoing = following.accepts_incoming(tokens, batch)
+                elif following.hands_off and layer.applies_following() and following.first_norm() is not None:
+                    outgoing = FollowingNorm(following.first_norm())
             layer.forward(x, batch, storage.kv[owner], storage.state[owner], reads_only=entry.cache_of is not None,
                           incoming=incoming, outgoing=outgoing)
             incoming = outgoing

@@ -33,11 +33,11 @@ MODULES: Dict[str, tuple] = {
     "elementwise": ("hip", ["kernels/elementwise.hip"], ["kernels/common.h"]),
     "gemm_generic": ("hip", ["kernels/gemm_generic.hip"], ["kernels/common.h"]),
     "attn_generic": ("hip", ["kernels/attn_generic.hip"], ["kernels/common.h", "kernels/attn_extras.h"]),
-    "heads": ("hip", ["kernels/heads.hip"], ["kernels/common.h"]),
+    "heads": ("hip", ["kernels/heads.hip"], ["kernels/common.h", "kernels/conv_state.h"]),
     "gemm_bf16": ("hip", ["kernels/gemm_bf16.hip"], ["kernels/common.h", "kernels/pipeline.h", "kernels/no_alloc.h"]),
     "sampling": ("hip", ["kernels/sampling.hip"], ["kernels/common.h"]),
     "recurrent": ("hip", ["kernels/recurrent.hip"], ["kernels/common.h"]),
-    "scan": ("hip", ["kernels/scan.hip"], ["kernels/common.h"]),
+    "scan": ("hip", ["kernels/scan.hip"], ["kernels/common.h", "kernels/conv_state.h"]),
     "state_space": ("hip", ["kernels/state_space.hip"], ["kernels/common.h"]),
     "streams": ("hip", ["kernels/streams.hip"], ["kernels/common.h"]),
     "latent": ("hip", ["kernels/latent.hip"], ["kernels/common.h", "kernels/group_tile.h"]),

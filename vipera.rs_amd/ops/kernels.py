@@ -1329,27 +1329,43 @@ def moe_route(logits: torch.Tensor, top: int, ids: torch.Tensor, weights: torch.
         _dev(correction)
         _need(mode == 3 and correction.dtype == torch.float32 and correction.is_contiguous()
               and correction.numel() == experts, "moe_route: one 32-bit correction per expert, with steered scores")
-    fn = _fn("moe", "vk_moe_route_steered", [_p, _i, _i, _i, _i, _i, _i, _i, _p, _f, _ll, _p, _p, _p, _p, _p, _p, _p])
+    fn = _fn("moe", "vk_moe_route", [_p, _i, _i, _i, _i, _i, _i, _i, _p, _f, _ll, _p, _p, _p, _p, _p, _p, _p])
     _status(fn(_ptr(logits), experts, top, tokens, tile_rows, int(groups), int(keep), mode, _ptr(correction),
                float(weight_scale), logits.stride(0) if tokens > 1 else experts, _ptr(ids), _ptr(weights), _ptr(offsets),
                _ptr(order), _ptr(tiles), _ptr(num_tiles), _stream()), "moe_route")
 
 
-def moe_experts(h: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, offsets: torch.Tensor,
+def moe_experts(h: torch.Tensor, w_gate: Optional[torch.Tensor], w_up: torch.Tensor, w_down: torch.Tensor, offsets: torch.Tensor,
                 order: torch.Tensor, tiles: torch.Tensor, num_tiles: torch.Tensor, weights: torch.Tensor, top: int,
                 limit: float, alpha: float, act: torch.Tensor, pair_out: torch.Tensor, residual: torch.Tensor,
-                accumulate: bool = True, weigh_input: bool = False) -> None:
+                accumulate: bool = True, weigh_input: bool = False, plain: Optional[str] = None,
+                extra: Optional[torch.Tensor] = None, extra_gate: Optional[torch.Tensor] = None,
+                stream: Optional[torch.Tensor] = None) -> None:
     """The chosen experts of every token: ``y = g * sigmoid(alpha * g) * (u + 1)`` with ``g = min(Wg h, limit)`` and
     ``u = clamp(Wu h, -limit, limit)``, or with an infinite ``limit`` ``y = g * sigmoid(alpha * g) * u`` (alpha 1:
     ``silu(g) * u``); then ``Wd y``; ``residual += sum_j weights[t, j] * expert_j(h[t])`` (without ``accumulate``: ``=``).
-    ``weigh_input``: ``residual += sum_j expert_j(weights[t, j] * h[t])`` instead."""
-    _dev(h, w_gate, w_up, w_down, offsets, order, tiles, num_tiles, weights, act, pair_out, residual)
+    ``weigh_input``: ``residual += sum_j expert_j(weights[t, j] * h[t])`` instead.  ``plain`` ("relu2", "silu" or
+    "gelu_tanh"): experts without a gate, ``Wd plain(Wu h)`` (``w_gate`` None).  ``extra`` ([tokens, width] 32-bit): joins the
+    sum, times ``sigmoid(extra_gate[t])`` if a gate ([tokens, >= 1] 32-bit, may be a view of some columns) is given.
+    ``stream`` ([tokens, width] bfloat16): receives the residual's new rows."""
+    _dev(h, w_gate, w_up, w_down, offsets, order, tiles, num_tiles, weights, act, pair_out, residual, extra, extra_gate, stream)
     tokens, width = h.shape
-    experts, ff, _ = w_gate.shape
-    _need(h.stride(1) == 1 and w_gate.shape == (experts, ff, width) and w_up.shape == w_gate.shape
+    experts, ff, _ = w_up.shape
+    _need((w_gate is None) == (plain is not None) and plain in (None, "relu2", "silu", "gelu_tanh"),
+          "moe_experts: experts with a gate, or an activation without one")
+    _need(h.stride(1) == 1 and w_up.shape == (experts, ff, width) and (w_gate is None or w_gate.shape == w_up.shape)
           and w_down.shape == (experts, width, ff), "moe_experts: weight shapes")
+    if extra is not None:
+        _f32(extra, "moe_experts: extra")
+        _need(extra.shape == (tokens, width) and extra.is_contiguous(), "moe_experts: extra")
+    if extra_gate is not None:
+        _f32s(extra_gate, "moe_experts: extra_gate")
+        _need(extra is not None and extra_gate.dim() == 2 and extra_gate.shape[0] == tokens, "moe_experts: extra_gate")
+    if stream is not None:
+        _need(stream.dtype == torch.bfloat16 and stream.shape == (tokens, width) and stream.is_contiguous(),
+              "moe_experts: stream")
     for t in (w_gate, w_up, w_down):
-        _need(t.dtype == h.dtype and t.is_contiguous(), "moe_experts: weights must be contiguous and of h's dtype")
+        _need(t is None or t.dtype == h.dtype and t.is_contiguous(), "moe_experts: weights must be contiguous and of h's dtype")
     _need(act.dtype == h.dtype and act.shape == (tokens * top, ff) and act.is_contiguous(), "moe_experts: act")
     _f32(pair_out, "moe_experts: pair_out")
     _f32(residual, "moe_experts: residual")
@@ -1360,11 +1376,13 @@ def moe_experts(h: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor, w_dow
     _need(offsets.numel() == experts + 1 and order.numel() == tokens * top
           and tiles.numel() >= 2 * moe_max_tiles(tokens * top, experts, moe_tile_rows(h, width, ff)),
           "moe_experts: grouping (made by moe_route with moe_tile_rows(h, width, ff))")
-    fn = _fn("moe", "vk_moe_experts_weighed", [_p, _ll, _p, _p, _p, _i, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _f, _f, _p, _p,
-                                               _p, _i, _i, _p])
+    fn = _fn("moe", "vk_moe_experts", [_p, _ll, _p, _p, _p, _i, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _f, _f, _i, _p, _p,
+                                       _p, _i, _i, _p, _p, _ll, _p, _p])
     _status(fn(_ptr(h), h.stride(0), _ptr(w_gate), _ptr(w_up), _ptr(w_down), _dt(h, "h"), _ptr(offsets), _ptr(order),
                _ptr(tiles), _ptr(num_tiles), _ptr(weights), tokens, experts, top, width, ff, float(limit), float(alpha),
-               _ptr(act), _ptr(pair_out), _ptr(residual), 1 if accumulate else 0, 1 if weigh_input else 0, _stream()),
+               ACTIVATIONS[plain] if plain else 0, _ptr(act), _ptr(pair_out), _ptr(residual), 1 if accumulate else 0,
+               1 if weigh_input else 0, _ptr(extra), _ptr(extra_gate), extra_gate.stride(0) if extra_gate is not None else 0,
+               _ptr(stream), _stream()),
             "moe_experts")
 
 
@@ -1376,11 +1394,17 @@ def _f32s(tensor: torch.Tensor, what: str) -> None:
 
 def rmsnorm_add(y: torch.Tensor, weight: torch.Tensor, eps: float, residual: torch.Tensor,
                 next_out: Optional[torch.Tensor] = None, next_weight: Optional[torch.Tensor] = None,
-                next_eps: float = 0.0) -> None:
+                next_eps: float = 0.0, next_kind: str = "rms", next_bias: Optional[torch.Tensor] = None) -> None:
     """``residual += y / sqrt(mean(y^2) + eps) * weight`` row by row, all 32-bit.  With ``next_out`` the new rows also
     leave as the next part's input, in its dtype: ``residual / sqrt(mean(residual^2) + next_eps) * next_weight`` (the
-    norm in front of the next sublayer), or the rows as they are without ``next_weight``."""
-    _dev(y, weight, residual, next_out, next_weight)
+    norm in front of the next sublayer; ``next_kind`` "layer": with the rows' means taken off first, and ``next_bias``
+    added if it is given), or the rows as they are without ``next_weight``."""
+    _dev(y, weight, residual, next_out, next_weight, next_bias)
+    _need(next_kind in ("rms", "layer") and (next_bias is None or (next_kind == "layer" and next_weight is not None)),
+          "rmsnorm_add: next_kind")
+    if next_bias is not None:
+        _need(next_bias.dtype == torch.float32 and next_bias.numel() == residual.shape[1] and next_bias.is_contiguous(),
+              "rmsnorm_add: next_bias")
     _f32(y, "rmsnorm_add: y")
     _f32(residual, "rmsnorm_add: residual")
     rows, width = residual.shape
@@ -1391,9 +1415,9 @@ def rmsnorm_add(y: torch.Tensor, weight: torch.Tensor, eps: float, residual: tor
     if next_weight is not None:
         _need(next_out is not None and next_weight.dtype == torch.float32 and next_weight.numel() == width
               and next_weight.is_contiguous(), "rmsnorm_add: next_weight")
-    fn = _fn("elementwise", "vk_rmsnorm_add", [_p, _p, _p, _i, _i, _f, _p, _f, _p, _i, _p])
-    _status(fn(_ptr(y), _ptr(weight), _ptr(residual), rows, width, float(eps), _ptr(next_weight), float(next_eps),
-               _ptr(next_out), _dt(next_out, "next_out") if next_out is not None else 0, _stream()), "rmsnorm_add")
+    fn = _fn("elementwise", "vk_rmsnorm_add", [_p, _p, _p, _i, _i, _f, _p, _p, _f, _i, _p, _i, _p])
+    _status(fn(_ptr(y), _ptr(weight), _ptr(residual), rows, width, float(eps), _ptr(next_weight), _ptr(next_bias),
+               float(next_eps), 1 if next_kind == "layer" else 0, _ptr(next_out), _dt(next_out, "next_out") if next_out is not None else 0, _stream()), "rmsnorm_add")
 
 
 def axpby(x: torch.Tensor, a: float, y: torch.Tensor, b: float, out: torch.Tensor, accumulate: bool = False) -> None:
@@ -1410,18 +1434,17 @@ ACTIVATIONS = {"none": 0, "relu2": 1, "silu": 2, "gelu_tanh": 3, "sigmoid": 4}
 
 
 def activation(x: torch.Tensor, kind: str, out: torch.Tensor, mul: Optional[torch.Tensor] = None) -> None:
-    """``out = act(x) (* mul)`` elementwise; ``x`` and ``mul`` may be row-strided views of either dtype, ``out`` is
-    contiguous.  ``kind``: none (a change of type), relu2 (the square of relu), silu, gelu_tanh, sigmoid."""
+    """``out = act(x) (* mul)`` elementwise; all three may be row-strided views of either dtype.  ``kind``: none (a change of type), relu2 (the square of relu), silu, gelu_tanh, sigmoid."""
     _dev(x, out, mul)
     _need(kind in ACTIVATIONS, f"activation: kind {kind!r}; known: {', '.join(ACTIVATIONS)}")
     rows, width = out.shape
-    _need(x.shape == out.shape and x.stride(1) == 1 and out.is_contiguous(), "activation: shapes")
+    _need(x.shape == out.shape and x.stride(1) == 1 and out.stride(1) == 1, "activation: shapes")
     if mul is not None:
         _need(mul.shape == out.shape and mul.stride(1) == 1, "activation: the factor's shape")
-    fn = _fn("elementwise", "vk_activation", [_p, _i, _ll, _p, _i, _ll, _p, _i, _i, _i, _i, _p])
+    fn = _fn("elementwise", "vk_activation", [_p, _i, _ll, _p, _i, _ll, _p, _i, _ll, _i, _i, _i, _p])
     _status(fn(_ptr(x), _dt(x, "x"), x.stride(0), _ptr(mul), _dt(mul, "mul") if mul is not None else 0,
-               mul.stride(0) if mul is not None else 0, _ptr(out), _dt(out, "out"), rows, width, ACTIVATIONS[kind],
-               _stream()), "activation")
+               mul.stride(0) if mul is not None else 0, _ptr(out), _dt(out, "out"), out.stride(0), rows, width,
+               ACTIVATIONS[kind], _stream()), "activation")
 
 
 def whole_norm_pack(proj: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor], eps: float,
@@ -1686,6 +1709,64 @@ def head_prepare(proj: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight:
                float(eps), _ptr(positions), _ptr(inv_freq), int(rot_dims), float(amplitude), tokens, heads, kv_heads, maps, dim,
                vdim, width, _ptr(qkv), _dt(qkv, "qkv"), _ptr(k_cache), _ptr(v_cache), _ptr(entry_of_token), _ptr(block_table),
                table_width, block_size, _stream()), "head_prepare")
+
+
+def head_conv_prepare(proj: torch.Tensor, conv: Optional[torch.Tensor], state: Optional[torch.Tensor],
+                      entry_of: torch.Tensor, entry_start: torch.Tensor, entry_first_pos: torch.Tensor, slots: torch.Tensor,
+                      num_entries: int, q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor], norm: bool,
+                      eps: float, positions: torch.Tensor, inv_freq: Optional[torch.Tensor], rot_dims: int, heads: int,
+                      kv_heads: int, dim: int, vdim: int, own_values: bool, width: int, q: torch.Tensor,
+                      k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
+                      angles: Optional[torch.Tensor] = None, amplitude: float = 1.0) -> None:
+    """The 32-bit sums ``proj`` = ``[q | k | (v) | ...]`` of a step's tokens: q and k pass a causal convolution over time per
+    channel (``conv [(heads + kv_heads) * dim, taps]``, the last column the current token's, or None) that goes on from the
+    request's row of ``state`` (``(taps - 1) * (heads + kv_heads) * dim`` floats, oldest input first; zeros at position 0) and
+    leaves the entry's last inputs there; then, with ``norm``, every head is divided by its root mean square and multiplied by
+    its weight of ``dim`` numbers (None: none), and its first ``rot_dims`` numbers are rotated (half-split pairs; ``angles``:
+    a step's table from :func:`rope_angles`, else sines and cosines times ``amplitude`` are computed from ``inv_freq``).
+    Queries go to ``q [tokens, heads * width]``, keys and values (``own_values``: columns of ``proj``; else the keys as
+    they leave the convolution) into the cache's pages only."""
+    _dev(proj, conv, state, entry_of, entry_start, entry_first_pos, slots, q_weight, k_weight, positions, inv_freq, q, k_cache,
+         v_cache, block_table, angles)
+    tokens, channels = proj.shape[0], (heads + kv_heads) * dim
+    _need(proj.dtype == torch.float32 and proj.dim() == 2 and proj.stride(1) == 1
+          and proj.shape[1] >= channels + (kv_heads * vdim if own_values else 0),
+          "head_conv_prepare: proj must be 32-bit [tokens, >= q + k (+ v) columns]")
+    _need(own_values or vdim == dim, "head_conv_prepare: values that are the keys have the keys' width")
+    _need(dim <= width and vdim <= width <= 256, "head_conv_prepare: the padded width holds every head, at most 256")
+    taps = 1
+    if conv is not None:
+        taps = conv.shape[1]
+        _need(conv.dtype == torch.float32 and conv.shape == (channels, taps) and conv.is_contiguous() and taps >= 1,
+              "head_conv_prepare: conv must be 32-bit [q + k channels, taps]")
+    if taps > 1:
+        _need(state is not None and state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1
+              and state.shape[1] >= (taps - 1) * channels, "head_conv_prepare: state row too short")
+    for weight in (q_weight, k_weight):
+        if weight is not None:
+            _need(weight.dtype == torch.float32 and weight.numel() == dim and weight.is_contiguous(), "head_conv_prepare: weights")
+    _i32(entry_of, entry_start, entry_first_pos, slots, positions)
+    _need(entry_of.numel() >= tokens and positions.numel() >= tokens, "head_conv_prepare: entries and positions")
+    _entries_ok((entry_start, entry_first_pos, slots), num_entries)
+    _need(rot_dims % 2 == 0 and 0 <= rot_dims <= dim, "head_conv_prepare: rot_dims")
+    if rot_dims:
+        _need(inv_freq is not None and inv_freq.dtype == torch.float32 and inv_freq.numel() == rot_dims // 2,
+              "head_conv_prepare: one frequency per rotated pair")
+    if angles is not None:
+        _need(angles.dtype == torch.float32 and angles.is_contiguous() and angles.numel() == tokens * rot_dims,
+              "head_conv_prepare: angles must be [tokens, rot_dims / 2, 2]")
+    _need(q.shape == (tokens, heads * width) and q.is_contiguous(), "head_conv_prepare: q shape")
+    _need(_cache_ok(k_cache, v_cache, kv_heads, width, q.dtype), "head_conv_prepare: cache shape or dtype")
+    _need(block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.is_contiguous()
+          and block_table.shape[0] >= num_entries, "head_conv_prepare: block table")
+    fn = _fn("heads", "vk_head_conv_prepare", [_p, _ll, _p, _i, _p, _ll, _p, _p, _p, _p, _i, _p, _p, _i, _f, _p, _p, _p, _i, _f,
+                                               _i, _i, _i, _i, _i, _i, _i, _p, _i, _p, _p, _p, _i, _i, _p])
+    _status(fn(_ptr(proj), proj.stride(0), _ptr(conv), taps, _ptr(state), state.stride(0) if state is not None else 0,
+               _ptr(entry_of), _ptr(entry_start), _ptr(entry_first_pos), _ptr(slots), num_entries, _ptr(q_weight),
+               _ptr(k_weight), 1 if norm else 0, float(eps), _ptr(positions), _ptr(inv_freq), _ptr(angles), int(rot_dims),
+               float(amplitude), tokens, heads, kv_heads, dim, vdim, 1 if own_values else 0, width, _ptr(q), _dt(q, "q"),
+               _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1], k_cache.shape[2], _stream()),
+            "head_conv_prepare")
 
 
 def head_finish(attn: torch.Tensor, out: torch.Tensor, heads: int, vdim: int, width: int, maps: int = 1,

@@ -25,6 +25,9 @@ to the scaled score by the distance between query and key: one row per distance 
 from there to ``far``, the last row from ``far`` on); ``maps: 2`` with ``diff`` (differential attention: q and k hold two
 maps per head, each an attention of its own over the same values; the head's output is ``a_1 - lambda a_2`` with
 ``lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff``, divided by its root mean square and multiplied by ``1 - diff``);
+``values: "keys"`` (the layer has no value projection: a key head, as projected and convolved, ahead of norm and rotation,
+is also its value head); ``conv`` (q and k pass a causal convolution of that many taps over time per channel, right behind
+the projection and its bias; the last inputs of a request are in its state row);
 ``tensors`` (the tensors' names after the part's name).  With any of these but the first three the step runs
 as one product ``[q | k | v | g]`` with 32-bit sums (biases added there), a kernel that norms and lays the heads out at
 one padded width, the rotation with the cache write, the paged attention kernels at that width, and a kernel that
@@ -43,8 +46,8 @@ from ..ops import kernels
 from ..ops.attention import AttentionExtras, paged_attention
 from ..ops.linear import linear, linear_follow, split_qkv_plan, streams_in_wave_order
 from ..weights.checkpoint import MATRIX, VECTOR, TensorSpec
-from .base import KVCacheSpec, Mixer, register_mixer
-from .rotary import pairs_apart
+from .base import KVCacheSpec, Mixer, StateSpec, register_mixer
+from .rotary import pairs_apart, prompt_angles
 
 
 def _cat(tensors: List[torch.Tensor]) -> torch.Tensor:
@@ -58,7 +61,7 @@ _DEFAULT_NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weigh
                   "g": "g_proj.weight", "q_norm": "q_norm.weight", "k_norm": "k_norm.weight",
                   "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias", "o_bias": "o_proj.bias",
                   "value_mix": "value_mix", "sink": "sink", "rel": "rel", "lq1": "lq1", "lk1": "lk1", "lq2": "lq2",
-                  "lk2": "lk2"}
+                  "lk2": "lk2", "q_conv": "q_conv", "k_conv": "k_conv"}
 
 VALUE_MIX_KEY = "attention.value_mix.source"    # where a step keeps the source layer's values (``batch.shared``)
 
@@ -71,8 +74,17 @@ def _tensor_names(p) -> Dict[str, str]:
 
 def _is_general(p) -> bool:
     """Whether the layer needs the path that norms, pads and gates (see the module's text)."""
-    return bool(p.get("qk_norm") or p.get("gate") or p.get("value_mix") or int(p.get("maps") or 1) > 1
+    return bool(p.get("qk_norm") or p.get("gate") or p.get("value_mix") or int(p.get("maps") or 1) > 1 or _convolves(p)
                 or int(p.get("value_dim") or p["head_dim"]) != int(p["head_dim"]))
+
+
+def _convolves(p) -> bool:
+    """Whether q and k go through the kernel that convolves them and takes values from keys."""
+    return p.get("values") == "keys" or bool(p.get("conv"))
+
+
+def _projections(p) -> str:
+    return "qk" if p.get("values") == "keys" else "qkv"
 
 
 def _padded_width(p) -> int:
@@ -128,6 +140,9 @@ class Attention(Mixer):
         if (self.qk_norm == "unit" or self.maps > 1) and self.value_mix:
             raise UnsupportedError("attention: value_mix beside qk_norm \"unit\" or several maps is not implemented")
         self.prepares = self.qk_norm != "whole" and not self.value_mix
+        self.convolves, self.own_values = _convolves(p), p.get("values") != "keys"
+        self.taps = int(p.get("conv") or 1)
+        self.w_conv = None
         self.extras = AttentionExtras(keep_first=self.keep_first)
         self.subtract = 0.0
         scale = p.get("scale")
@@ -136,6 +151,8 @@ class Attention(Mixer):
             raise InvalidArgumentError(f"heads {self.heads} is not a multiple of kv_heads {self.kv_heads}")
         self.q_width = self.heads * self.maps * self.head_dim
         self.kv_width = self.kv_heads * self.maps * self.head_dim
+        # where the gate's columns begin in the one product
+        self.gate_col = self.q_width + self.kv_width + (self.kv_heads * self.value_dim if self.own_values else 0)
         self.w_qkv = self.b_qkv = self.w_o = self.b_o = self.q_norm = self.k_norm = self.mix = None
 
     @classmethod
@@ -149,9 +166,13 @@ class Attention(Mixer):
         q, kv = int(p["heads"]) * maps * hd, int(p["kv_heads"]) * maps * hd
         specs: List[TensorSpec] = []
         for name, rows in (("q", q), ("k", kv), ("v", int(p["kv_heads"]) * vd)):
+            if name not in _projections(p):
+                continue
             specs.append(TensorSpec(base + names[name], (rows, hidden), MATRIX))
             if p.get("qkv_bias"):
                 specs.append(TensorSpec(base + names[name + "_bias"], (rows,), VECTOR))
+            if name != "v" and p.get("conv"):
+                specs.append(TensorSpec(base + names[name + "_conv"], (rows, int(p["conv"])), VECTOR, std=0.5))
         specs.append(TensorSpec(base + names["o"], (hidden, int(p["heads"]) * vd), MATRIX))
         if p.get("out_bias"):
             specs.append(TensorSpec(base + names["o_bias"], (hidden,), VECTOR))
@@ -179,7 +200,8 @@ class Attention(Mixer):
     def load(self, tensors: Dict[str, torch.Tensor]) -> None:
         base = f"{self.prefix}{self.spec.params['name']}."
         names = _tensor_names(self.spec.params)
-        parts = [tensors[base + names[n]] for n in "qkv"]
+        projections = _projections(self.spec.params)
+        parts = [tensors[base + names[n]] for n in projections]
         if self.spec.params.get("pairs") == "interleaved":
             rotary_dim = int(self.spec.params["rotary_dim"])
             parts[0] = pairs_apart(parts[0], self.heads * self.maps, self.head_dim, 0, rotary_dim)
@@ -188,10 +210,12 @@ class Attention(Mixer):
             parts.append(tensors[base + names["g"]])
         self.w_qkv = _cat(parts)
         if self.qkv_bias:
-            biases = [tensors[base + names[n + "_bias"]] for n in "qkv"]
+            biases = [tensors[base + names[n + "_bias"]] for n in projections]
             if self.gate:   # the gate's rows of the one product have no bias
                 biases.append(torch.zeros(parts[-1].shape[0], dtype=biases[0].dtype, device=biases[0].device))
             self.b_qkv = torch.cat(biases).contiguous()
+        if self.spec.params.get("conv"):
+            self.w_conv = torch.cat([tensors[base + names[n]] for n in ("q_conv", "k_conv")]).contiguous()
         self.w_o = tensors[base + names["o"]]
         if self.out_bias:
             self.b_o = tensors[base + names["o_bias"]]
@@ -218,7 +242,11 @@ class Attention(Mixer):
         # pool is sized for whole requests
         # kept first positions lie outside the window that the pool's bookkeeping knows: such a layer keeps everything
         window = 0 if p.get("keep_first") else int(p.get("window") or 0)
-        return KVCacheSpec(int(p["kv_heads"]), _padded_width(p), window), None
+        state, taps = None, int(p.get("conv") or 1)
+        if taps > 1:
+            channels = (int(p["heads"]) + int(p["kv_heads"])) * int(p["head_dim"])
+            state = StateSpec(((taps - 1) * channels,), torch.float32)
+        return KVCacheSpec(int(p["kv_heads"]), _padded_width(p), window), state
 
     @classmethod
     def check_supported(cls, spec: PartSpec, dtype: torch.dtype) -> None:
@@ -228,6 +256,14 @@ class Attention(Mixer):
             raise UnsupportedError(f"attention: pairs {p.get('pairs')!r}; \"interleaved\" or none")
         if p.get("pairs") and (p.get("qk_norm") in ("whole", "head") or p.get("qkv_bias")):
             raise UnsupportedError("attention: interleaved pairs beside weights of q and k norms or biases are not implemented")
+        if p.get("values") not in (None, "keys"):
+            raise UnsupportedError(f"attention: values {p.get('values')!r}; \"keys\" or none")
+        if _convolves(p) and (p.get("qk_norm") not in (None, "head") or p.get("value_mix") or p.get("pairs")
+                              or int(p.get("maps") or 1) > 1):
+            raise UnsupportedError("attention: convolved queries and keys, or values that are the keys, beside qk_norm "
+                                   f"{p.get('qk_norm')!r}, value_mix, interleaved pairs or several maps are not implemented")
+        if p.get("values") == "keys" and int(p.get("value_dim") or p["head_dim"]) != int(p["head_dim"]):
+            raise InvalidArgumentError("attention: values that are the keys have the keys' width")
         if p.get("qk_norm") not in (None, "whole", "head", "unit"):
             raise UnsupportedError(f"attention: qk_norm {p.get('qk_norm')!r} is not implemented; \"whole\", \"head\", "
                                    "\"unit\" or none")
@@ -278,7 +314,7 @@ class Attention(Mixer):
         # the fused products can divide by the norm themselves
         return self._fused(tokens, position, batch) is not None
 
-    def _forward_general(self, h, batch, cache, position, residual, reads_only: bool, accumulate: bool) -> None:
+    def _forward_general(self, h, batch, cache, state, position, residual, reads_only: bool, accumulate: bool) -> None:
         """q and k normed over the whole projection, values of another width, a gate on the output: see the module's
         text.  Heads are ``padded`` wide in the buffers that the rotation and the attention kernels see."""
         tokens = residual.shape[0]
@@ -286,7 +322,8 @@ class Attention(Mixer):
         proj = torch.empty((tokens, self.w_qkv.shape[0]), dtype=torch.float32, device=residual.device)
         linear(h, self.w_qkv, self.b_qkv, proj)
         heads = self.heads * self.maps            # query heads as the attention kernels count them
-        qkv = self.runtime.empty((tokens, (heads + 2 * self.kv_heads) * width))
+        # the attention kernels read queries by row; keys and values come from the cache
+        qkv = self.runtime.empty((tokens, (heads if self.convolves else heads + 2 * self.kv_heads) * width))
         eps = float(self.spec.params.get("eps") or 0.0)
         first = None
         if self.value_mix:
@@ -302,7 +339,17 @@ class Attention(Mixer):
                                                "before it in the run order keeps values of this shape")
         fused = position.fused_rotary()
         inv_freq, rotary_dim = fused if fused is not None else (None, 0)
-        if self.prepares:
+        if self.convolves:
+            if fused is None or reads_only:
+                raise UnsupportedError("attention: convolved queries and keys need a rotation the kernels know, or none, and a "
+                                       "cache of their own")
+            kernels.head_conv_prepare(proj, self.w_conv, state, batch.entry_of_token, batch.entry_start, batch.entry_first_pos,
+                                      batch.slots, batch.num_entries, self.q_norm, self.k_norm, bool(self.qk_norm), eps,
+                                      batch.positions, inv_freq, rotary_dim, self.heads, self.kv_heads, self.head_dim,
+                                      self.value_dim, self.own_values, width, qkv, cache.k, cache.v,
+                                      batch.block_tables[cache.group], prompt_angles(position, batch, rotary_dim),
+                                      position.amplitude)
+        elif self.prepares:
             if fused is None:
                 raise UnsupportedError("attention: qk_norm \"unit\" and several maps need a rotation the kernels know, or none")
             # rotation, norm, layout and the cache write in one pass
@@ -337,7 +384,7 @@ class Attention(Mixer):
             linear(attn, self.w_o, self.b_o, residual, accumulate=accumulate)
             return
         values = self.runtime.empty((tokens, self.heads * self.value_dim))
-        gate = proj[:, self.q_width + self.kv_width + self.kv_heads * self.value_dim:] if self.gate else None
+        gate = proj[:, self.gate_col:] if self.gate else None
         if self.maps > 1 or self.gate == "head_sigmoid":
             kernels.head_finish(attn, values, self.heads, self.value_dim, width, self.maps, self.subtract,
                                 unit_norm=self.maps > 1, eps=eps, factor=1.0 - self.diff if self.maps > 1 else 1.0,
@@ -350,7 +397,7 @@ class Attention(Mixer):
                 incoming=None, accumulate: bool = True) -> None:
         tokens = residual.shape[0]
         if self.general:
-            return self._forward_general(h, batch, cache, position, residual, reads_only, accumulate)
+            return self._forward_general(h, batch, cache, state, position, residual, reads_only, accumulate)
         how = self._fused(tokens, position, batch)
         if incoming is not None and how is None:
             raise UnsupportedError("attention was handed a split norm for a step whose product cannot divide by it")

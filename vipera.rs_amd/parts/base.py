@@ -25,6 +25,9 @@ embedding             ``embed(batch) -> x``: the 32-bit residual ``[tokens, widt
                       (the batch brings tokens and positions); ``reads_device_tokens`` says whether it
                       takes token ids that the sampler left on the device (``batch.token_source``).
 head                  ``forward(h) -> logits`` (32-bit) and ``vocab``.
+rejoin                ``keep(x, batch)`` takes the embedding's output once a step, ahead of the first layer;
+                      ``forward(x, batch)`` then
+                      joins the stream ``x`` with it, in place, ahead of every run-order entry with ``rejoins``.
 """
 from __future__ import annotations
 
@@ -111,6 +114,14 @@ class NormHandoff:
     groups: int = 0
 
 
+@dataclass
+class FollowingNorm:
+    """The next layer's first norm, for the last part of the layer before it to apply to the rows it leaves: it sets
+    ``out`` to the norm's output of the new rows, or leaves it None, and the norm runs as a kernel of its own."""
+    norm: "Norm"
+    out: Optional[torch.Tensor] = None
+
+
 class Norm(Part):
     def forward(self, x: torch.Tensor, out: Optional[torch.Tensor] = None,
                 rows: Optional[torch.Tensor] = None) -> torch.Tensor:
@@ -184,6 +195,13 @@ class FeedForward(Part):
     #: as :attr:`Mixer.can_overwrite`
     can_overwrite = False
 
+    #: a feed-forward that sets this takes ``stream=`` in ``forward``, a buffer of the residual's shape in the run's dtype,
+    #: and leaves the new rows of the residual in it
+    leaves_stream = False
+
+    #: a part that sets this takes ``following=`` (a :class:`FollowingNorm`) in ``forward`` and may fill it
+    applies_following = False
+
     #: a feed-forward that sets this takes ``outgoing=`` in ``forward`` and may fill it for the next layer's first norm
     fills_handoff = False
 
@@ -223,6 +241,15 @@ class Block:
     #: first norm prepared by this one)
     hands_off = False
 
+    def first_norm(self) -> Optional["Norm"]:
+        """The norm that reads the stream first, if the layer before may apply it (``forward`` then gets it as a
+        :class:`FollowingNorm` under ``incoming``), else None."""
+        return None
+
+    def applies_following(self) -> bool:
+        """Whether ``forward`` takes a :class:`FollowingNorm` under ``outgoing``."""
+        return False
+
     def forward(self, x, batch, cache, state, reads_only: bool = False) -> None:
         raise NotImplementedError
 
@@ -230,6 +257,7 @@ class Block:
 # --- registries ---------------------------------------------------------------------------------
 _REGISTRIES: Dict[str, Dict[str, type]] = {
     "mixer": {}, "ffn": {}, "norm": {}, "position": {}, "block": {}, "embedding": {}, "head": {},
+    "rejoin": {},
 }
 
 
@@ -268,6 +296,10 @@ def register_block(kind: str, cls: Type[Block]) -> None:
 
 def register_embedding(kind: str, cls: Type[Part]) -> None:
     _register("embedding", kind, cls)
+
+
+def register_rejoin(kind: str, cls: Type[Part]) -> None:
+    _register("rejoin", kind, cls)
 
 
 def register_head(kind: str, cls: Type[Part]) -> None:

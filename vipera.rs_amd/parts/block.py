@@ -1,7 +1,8 @@
 """Arrangements of a layer's parts.
 
 ``prenorm``: ``x += mixer(norm_1(x)); x += ffn(norm_2(x))``, the pre-norm residual block of the
-reference (crates/vipera-backend-cpu/src/model.rs:3-4, 975-1198).
+reference (crates/vipera-backend-cpu/src/model.rs:3-4, 975-1198); without a feed-forward (kind ``none``) the first half
+alone, and optionally a part that adds to the stream after both (``extras["after"]``, of the feed-forward family).
 ``parallel``: ``h = norm(x); x += mixer(h) + ffn(h)``; with a second norm of its own for the feed-forward,
 ``x += m * (mixer(norm_1(x)) + ffn(norm_2(x)))``, both norms of the same ``x``, ``m`` = ``params["residual_mult"]``.
 ``sandwich_norm``: a norm before and behind each sublayer, ``x += norm_1b(mixer(norm_1(x))); x += norm_2b(ffn(norm_2(x)))``,
@@ -14,32 +15,49 @@ from __future__ import annotations
 
 from typing import List
 
+import torch
+
 from ..config.base import LayerSpec
 from ..weights.checkpoint import TensorSpec
-from .base import Block, part_class, register_block
+from .base import Block, FollowingNorm, part_class, register_block
 
 
 class PreNormBlock(Block):
     def __init__(self, spec: LayerSpec, runtime):
         super().__init__(spec, runtime)
-        self.mixer_norm = part_class("norm", spec.mixer_norm.kind)(spec.mixer_norm, spec.prefix, runtime)
-        self.mixer = part_class("mixer", spec.mixer.kind)(spec.mixer, spec.prefix, runtime)
-        self.ffn_norm = part_class("norm", spec.ffn_norm.kind)(spec.ffn_norm, spec.prefix, runtime)
-        self.ffn = part_class("ffn", spec.ffn.kind)(spec.ffn, spec.prefix, runtime)
-        self.position = part_class("position", spec.position.kind)(spec.position, spec.prefix, runtime)
+        self.parts = {role: part_class(family, part.kind)(part, spec.prefix, runtime)
+                      for role, family, part in self._roles(spec)}
+        self.mixer_norm, self.mixer, self.position = (self.parts[role] for role in ("mixer_norm", "mixer", "position"))
+        self.ffn_norm, self.ffn, self.after = (self.parts.get(role) for role in ("ffn_norm", "ffn", "after"))
+
+    @classmethod
+    def _roles(cls, spec: LayerSpec):
+        roles = [("mixer_norm", "norm", spec.mixer_norm), ("mixer", "mixer", spec.mixer)]
+        if spec.ffn.kind != "none":
+            roles += [("ffn_norm", "norm", spec.ffn_norm), ("ffn", "ffn", spec.ffn)]
+        roles.append(("position", "position", spec.position))
+        if "after" in spec.extras:
+            roles.append(("after", "ffn", spec.extras["after"]))
+        return roles
 
     @classmethod
     def declare(cls, spec: LayerSpec) -> List[TensorSpec]:
         out: List[TensorSpec] = []
-        out += part_class("norm", spec.mixer_norm.kind).declare(spec.mixer_norm, spec.prefix)
-        out += part_class("mixer", spec.mixer.kind).declare(spec.mixer, spec.prefix)
-        out += part_class("norm", spec.ffn_norm.kind).declare(spec.ffn_norm, spec.prefix)
-        out += part_class("ffn", spec.ffn.kind).declare(spec.ffn, spec.prefix)
-        out += part_class("position", spec.position.kind).declare(spec.position, spec.prefix)
+        for _, family, part in cls._roles(spec):
+            out += part_class(family, part.kind).declare(part, spec.prefix)
+        if spec.ffn.kind == "none":
+            # a layer without a feed-forward does not read the norm in front of it; a folder may hold it all the same
+            out += [TensorSpec(t.name, t.shape, t.role, t.init, t.std, True)
+                    for t in part_class("norm", spec.ffn_norm.kind).declare(spec.ffn_norm, spec.prefix)]
         return out
 
+    @classmethod
+    def check_supported(cls, spec: LayerSpec, dtype) -> None:
+        for _, family, part in cls._roles(spec):
+            part_class(family, part.kind).check_supported(part, dtype)
+
     def load(self, tensors) -> None:
-        for part in (self.mixer_norm, self.mixer, self.ffn_norm, self.ffn, self.position):
+        for part in self.parts.values():
             part.load(tensors)
 
     hands_off = True
@@ -51,31 +69,48 @@ class PreNormBlock(Block):
         return self.mixer_norm.handoff(tokens)
 
     def fills_outgoing(self) -> bool:
-        return self.ffn.fills_handoff
+        return self.after is None and self.ffn is not None and self.ffn.fills_handoff
+
+    def first_norm(self):
+        return self.mixer_norm
+
+    def applies_following(self) -> bool:
+        return self.after is not None and self.after.applies_following
 
     def forward(self, x, batch, cache, state, reads_only: bool = False, incoming=None, outgoing=None) -> None:
         """With a few tokens a norm may be split between the product before it and the product after it, if all
         three can (see NormHandoff); otherwise it is a kernel of its own. ``incoming``: this block's first norm,
         filled by the layer before (``groups`` > 0) or not; ``outgoing``: the next layer's first norm, for this
-        block's feed-forward to fill."""
-        if incoming is not None and incoming.groups:
+        block's feed-forward to fill.  Behind a layer that ends in a part which applies the norm that follows, either is
+        a :class:`FollowingNorm` instead."""
+        mixer_kwargs = {}
+        if isinstance(incoming, FollowingNorm):
+            h = incoming.out if incoming.out is not None else self.mixer_norm.forward(x)
+        elif incoming is not None and incoming.groups:
             h = None
             mixer_kwargs = {"incoming": incoming}
         else:
             h = self.mixer_norm.forward(x)
-            mixer_kwargs = {}
         between = None
-        if self.mixer.fills_handoff and self.ffn.accepts_handoff(x.shape[0]):
+        if self.ffn is not None and self.mixer.fills_handoff and self.ffn.accepts_handoff(x.shape[0]):
             between = self.ffn_norm.handoff(x.shape[0])
             if between is not None:
                 mixer_kwargs["handoff"] = between
         self.mixer.forward(h, batch, cache, state, self.position, x, reads_only, **mixer_kwargs)
-        ffn_kwargs = {"outgoing": outgoing} if outgoing is not None and self.ffn.fills_handoff else {}
-        if between is not None and between.groups:
-            self.ffn.forward(None, batch, x, handoff=between, **ffn_kwargs)
-        else:
-            h = self.ffn_norm.forward(x)
-            self.ffn.forward(h, batch, x, **ffn_kwargs)
+        stream = None
+        if self.ffn is not None:
+            ffn_kwargs = {"outgoing": outgoing} if self.after is None and outgoing is not None and self.ffn.fills_handoff else {}
+            if self.after is not None and self.ffn.leaves_stream and getattr(self.after, "reads_stream_input", False) \
+                    and self.runtime.dtype != torch.float32:
+                stream = ffn_kwargs["stream"] = self.runtime.empty(tuple(x.shape))
+            if between is not None and between.groups:
+                self.ffn.forward(None, batch, x, handoff=between, **ffn_kwargs)
+            else:
+                h = self.ffn_norm.forward(x)
+                self.ffn.forward(h, batch, x, **ffn_kwargs)
+        if self.after is not None:
+            after_kwargs = {"following": outgoing} if isinstance(outgoing, FollowingNorm) and self.after.applies_following else {}
+            self.after.forward(stream, batch, x, **after_kwargs)
 
 
 class ParallelBlock(Block):
@@ -140,7 +175,6 @@ class ParallelBlock(Block):
             self.mixer.forward(h, batch, cache, state, self.position, x, reads_only)
             self.ffn.forward(h_ffn, batch, x)
             return
-        import torch
         from ..ops import kernels
         if self.mixer.can_overwrite:
             y = torch.empty_like(x)
@@ -199,7 +233,6 @@ class SandwichBlock(Block):
             part.load(tensors)
 
     def forward(self, x, batch, cache, state, reads_only: bool = False) -> None:
-        import torch
         parts = self.parts
         h = parts["mixer_norm"].forward(x)
         if parts["mixer"].can_overwrite:
@@ -273,7 +306,6 @@ class PostNormBlock(Block):
                 part.load(tensors)
 
     def _as_input(self, x, batch):
-        import torch
         from ..ops import kernels
         left = batch.shared.pop(self.STREAM_KEY, None)
         if left is not None and left[0] is x:
@@ -285,7 +317,6 @@ class PostNormBlock(Block):
         return h
 
     def _sublayer(self, run, part, x):
-        import torch
         if part.can_overwrite:
             y = torch.empty_like(x)
             run(y, {"accumulate": False})

@@ -106,6 +106,7 @@ class TokenSide(FeedForward):
     ``dim``, ``index``, ``eps``, ``activation`` ("gelu_tanh" unless given), ``name``; tensors ``<name>.gate | proj | norm``."""
 
     reads_stream_input = True     # forward's ``h`` may be the residual itself in the run's dtype
+    applies_following = True
 
     def __init__(self, spec: PartSpec, prefix: str, runtime):
         super().__init__(spec, prefix, runtime)
@@ -126,7 +127,7 @@ class TokenSide(FeedForward):
         base = f"{self.prefix}{self.spec.params['name']}."
         self.w_gate, self.w_proj, self.norm = tensors[base + "gate"], tensors[base + "proj"], tensors[base + "norm"]
 
-    def forward(self, h, batch, residual, **_unused) -> None:
+    def forward(self, h, batch, residual, following=None, **_unused) -> None:
         tokens = residual.shape[0]
         rows = batch.shared.get(SIDE_ROWS)
         if rows is None or rows.shape[1] < (self.index + 1) * self.dim:
@@ -141,7 +142,13 @@ class TokenSide(FeedForward):
         kernels.activation(gate, self.activation, gated, mul=rows[:, self.index * self.dim:(self.index + 1) * self.dim])
         y = torch.empty((tokens, self.hidden), dtype=torch.float32, device=residual.device)
         linear(gated, self.w_proj, None, y)
-        kernels.rmsnorm_add(y, self.norm, self.eps, residual)
+        fused = following.norm.as_kernel() if following is not None else None
+        if fused is None or fused[0] == "none":
+            kernels.rmsnorm_add(y, self.norm, self.eps, residual)
+            return
+        kind, weight, bias, eps = fused
+        following.out = self.runtime.empty((tokens, self.hidden))
+        kernels.rmsnorm_add(y, self.norm, self.eps, residual, following.out, weight, eps, next_kind=kind, next_bias=bias)
 
 
 class LMHead(Part):

@@ -14,6 +14,8 @@ expert, tensor ``<name>.correction``, that steers the choice and nothing else) a
 adds the sum of ``expert(w h)``.  ``shared``: a gated feed-forward of that width (``silu(Wg h) * (Wu h)`` through
 ``Wd``, tensors ``<name>.shared.gate | up | down``) that every token runs beside its experts; with ``shared_gate``
 ("sigmoid") its output is multiplied by ``sigmoid(Wsg h)``, one number per token (tensor ``<name>.shared.sg``).
+``form: "plain"``: the experts, the shared one too, have no gate, ``W_down act(W_up h)`` with ``activation`` ("relu2": the
+square of relu; "silu"; "gelu_tanh").  ``router_bias`` (a tensor's name after the part's): added to the router logits.
 
 The step's (token, choice) pairs are grouped by expert on the device, so nothing about the routing reaches the
 host and a step of single tokens can be captured; see ``csrc/kernels/moe.hip``.
@@ -29,14 +31,15 @@ from ..errors import InvalidArgumentError, UnsupportedError
 from ..ops import kernels
 from ..ops.linear import linear
 from ..weights.checkpoint import MATRIX, VECTOR, TensorSpec
-from .base import FeedForward, register_ffn
+from .base import FeedForward, part_class, register_ffn
 
 
 class MixtureOfExperts(FeedForward):
     """``params``: ``hidden``, ``intermediate`` (an expert's width), ``experts``, ``top``, ``limit`` (None: no clamp),
     ``alpha`` (1.702 unless given), ``groups`` and ``keep`` (1 and 1 unless given), ``scores`` ("chosen", "all" or
-    "sigmoid"), ``weigh`` ("output" or "input"), ``shared`` (the shared expert's width, or None), ``name``; tensors
-    ``<name>.router``, ``<name>.e<i>.gate | up | down`` and ``<name>.shared.gate | up | down``."""
+    "sigmoid"), ``weigh`` ("output" or "input"), ``shared`` (the shared expert's width, or None), ``form`` ("gated" or
+    "plain"), ``activation`` (of the plain form), ``router_bias``, ``name``; tensors ``<name>.router``,
+    ``<name>.e<i>.gate | up | down`` and ``<name>.shared.gate | up | down``."""
 
     def __init__(self, spec: PartSpec, prefix: str, runtime):
         super().__init__(spec, prefix, runtime)
@@ -49,18 +52,22 @@ class MixtureOfExperts(FeedForward):
         self.all_scores = {"chosen": False, "all": True, "sigmoid": "sigmoid", "steered": "steered"}[p.get("scores", "chosen")]
         self.weight_scale = float(p.get("weight_scale", 1.0))
         self.shared_gate = p.get("shared_gate")
-        self.correction = self.w_shared_gate = None
+        self.correction = self.w_shared_gate = self.b_router = None
+        self.plain = p.get("activation", "relu2") if p.get("form") == "plain" else None
         self.weigh_input = p.get("weigh", "output") == "input"
         self.shared = None
         if p.get("shared"):
-            from .mlp import GatedMLP
-            self.shared = GatedMLP(self._shared_spec(p), prefix, runtime)
+            shared = self._shared_spec(p)
+            self.shared = part_class("ffn", shared.kind)(shared, prefix, runtime)
         if not 1 <= self.top <= self.experts:
             raise InvalidArgumentError(f"a token cannot use {self.top} of {self.experts} experts")
         self.w_router = self.w_gate = self.w_up = self.w_down = None
 
     @staticmethod
     def _shared_spec(p) -> PartSpec:
+        if p.get("form") == "plain":
+            return PartSpec("mlp", {"hidden": int(p["hidden"]), "intermediate": int(p["shared"]),
+                                    "activation": p.get("activation", "relu2"), "name": f"{p['name']}.shared"})
         return PartSpec("gated_mlp", {"hidden": int(p["hidden"]), "intermediate": int(p["shared"]),
                                       "name": f"{p['name']}.shared",
                                       "tensors": {"gate": "gate", "up": "up", "down": "down"}})
@@ -72,15 +79,18 @@ class MixtureOfExperts(FeedForward):
         hidden, inter = int(p["hidden"]), int(p["intermediate"])
         specs = []
         for e in range(int(p["experts"])):
-            specs += [TensorSpec(f"{base}e{e}.gate", (inter, hidden), MATRIX),
-                      TensorSpec(f"{base}e{e}.up", (inter, hidden), MATRIX),
+            if p.get("form") != "plain":
+                specs.append(TensorSpec(f"{base}e{e}.gate", (inter, hidden), MATRIX))
+            specs += [TensorSpec(f"{base}e{e}.up", (inter, hidden), MATRIX),
                       TensorSpec(f"{base}e{e}.down", (hidden, inter), MATRIX)]
         specs.append(TensorSpec(base + "router", (int(p["experts"]), hidden), MATRIX))
+        if p.get("router_bias"):
+            specs.append(TensorSpec(base + p["router_bias"], (int(p["experts"]),), VECTOR, std=0.1))
         if p.get("scores") == "steered":
             specs.append(TensorSpec(base + "correction", (int(p["experts"]),), VECTOR, std=0.1))
         if p.get("shared"):
-            from .mlp import GatedMLP
-            specs += GatedMLP.declare(cls._shared_spec(p), prefix)
+            shared = cls._shared_spec(p)
+            specs += part_class("ffn", shared.kind).declare(shared, prefix)
             if p.get("shared_gate"):
                 specs.append(TensorSpec(base + "shared.sg", (1, hidden), MATRIX))
         return specs
@@ -101,6 +111,10 @@ class MixtureOfExperts(FeedForward):
         if spec.params.get("scores", "chosen") not in ("chosen", "all", "sigmoid", "steered"):
             raise UnsupportedError(f"mixture of experts: scores {spec.params.get('scores')!r}; \"chosen\", \"all\", "
                                    "\"sigmoid\" or \"steered\"")
+        if spec.params.get("form", "gated") not in ("gated", "plain") or (
+                spec.params.get("form") == "plain" and spec.params.get("activation", "relu2") not in ("relu2", "silu", "gelu_tanh")):
+            raise UnsupportedError(f"mixture of experts: form {spec.params.get('form')!r} with activation "
+                                   f"{spec.params.get('activation')!r}; \"gated\", or \"plain\" with relu2, silu or gelu_tanh")
         if spec.params.get("shared_gate") not in (None, "sigmoid"):
             raise UnsupportedError(f"mixture of experts: shared_gate {spec.params.get('shared_gate')!r}; \"sigmoid\" or none")
         if spec.params.get("weigh", "output") not in ("output", "input"):
@@ -110,7 +124,8 @@ class MixtureOfExperts(FeedForward):
         base = f"{self.prefix}{self.spec.params['name']}."
         dtype = self.runtime.dtype
         stack = lambda kind: torch.stack([tensors[f"{base}e{e}.{kind}"].to(dtype) for e in range(self.experts)]).contiguous()
-        self.w_gate, self.w_up, self.w_down = stack("gate"), stack("up"), stack("down")
+        self.w_gate = stack("gate") if self.plain is None else None
+        self.w_up, self.w_down = stack("up"), stack("down")
         self.w_router = tensors[base + "router"]
         if self.all_scores == "steered":
             self.correction = tensors[base + "correction"]
@@ -120,15 +135,20 @@ class MixtureOfExperts(FeedForward):
                 # the gate's row rides behind the router's rows: one product for all that is one number per token
                 self.w_shared_gate = tensors[base + "shared.sg"]
                 self.w_router = torch.cat([self.w_router.to(self.w_shared_gate.dtype), self.w_shared_gate]).contiguous()
+        if self.spec.params.get("router_bias"):
+            bias = torch.zeros(self.w_router.shape[0], dtype=torch.float32, device=self.w_router.device)
+            bias[:self.experts] = tensors[base + self.spec.params["router_bias"]].float()
+            self.b_router = bias
 
     can_overwrite = True
+    leaves_stream = True
 
-    def forward(self, h, batch, residual, accumulate: bool = True, **_unused) -> None:
+    def forward(self, h, batch, residual, accumulate: bool = True, stream=None, **_unused) -> None:
         tokens = residual.shape[0]
         device = residual.device
         pairs = tokens * self.top
         rows = torch.empty((tokens, self.w_router.shape[0]), dtype=torch.float32, device=device)
-        linear(h, self.w_router, None, rows)
+        linear(h, self.w_router, self.b_router, rows)
         logits = rows[:, :self.experts]
         tile_rows = kernels.moe_tile_rows(h, self.hidden, self.inter)
         ints = torch.empty(2 * pairs + self.experts + 2 + 2 * kernels.moe_max_tiles(pairs, self.experts, tile_rows),
@@ -143,15 +163,19 @@ class MixtureOfExperts(FeedForward):
                           weight_scale=self.weight_scale)
         act = self.runtime.empty((pairs, self.inter))
         pair_out = torch.empty((pairs, self.hidden), dtype=torch.float32, device=device)
-        kernels.moe_experts(h, self.w_gate, self.w_up, self.w_down, offsets, order, tiles, num_tiles, weights,
-                            self.top, self.limit, self.alpha, act, pair_out, residual, accumulate, self.weigh_input)
-        if self.shared is not None and self.w_shared_gate is None:
-            self.shared.forward(h, batch, residual)
-        elif self.shared is not None:
+        extra = None
+        if self.shared is not None and self.w_shared_gate is not None:
             # the shared expert into a buffer of its own, which joins the others' sum times the token's gate
-            own = torch.empty_like(residual)
-            self.shared.forward(h, batch, own, accumulate=False)
-            kernels.row_gate_add(own, rows[:, self.experts:], self.shared_gate, residual)
+            extra = torch.empty_like(residual)
+            self.shared.forward(h, batch, extra, accumulate=False)
+        elif self.shared is not None:
+            # its output lies in the residual already when the experts' sum joins
+            self.shared.forward(h, batch, residual, accumulate=accumulate)
+            accumulate = True
+        kernels.moe_experts(h, self.w_gate, self.w_up, self.w_down, offsets, order, tiles, num_tiles, weights,
+                            self.top, self.limit, self.alpha, act, pair_out, residual, accumulate, self.weigh_input,
+                            plain=self.plain, extra=extra, extra_gate=rows[:, self.experts:] if extra is not None else None,
+                            stream=stream)
 
 
 register_ffn("moe", MixtureOfExperts)

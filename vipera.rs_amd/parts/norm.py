@@ -84,7 +84,8 @@ class RMSNorm(Norm):
 
 class LayerNorm(Norm):
     """Layer norm: ``out = (x - mean) / sqrt(mean((x - mean)^2) + eps) * weight + bias``, all in 32-bit.  ``params``:
-    ``width``, ``eps``, ``tensor`` (the weight's name after the part's prefix; the bias is ``<tensor>.b``)."""
+    ``width``, ``eps``, ``tensor`` (the weight's name after the part's prefix; the bias is ``<tensor>.b``), ``bias`` (False:
+    there is none)."""
 
     def __init__(self, spec: PartSpec, prefix: str, runtime):
         super().__init__(spec, prefix, runtime)
@@ -94,7 +95,10 @@ class LayerNorm(Norm):
     @classmethod
     def declare(cls, spec: PartSpec, prefix: str) -> List[TensorSpec]:
         name, width = f"{prefix}{spec.params['tensor']}", int(spec.params["width"])
-        return [TensorSpec(name, (width,), VECTOR, "one_plus_normal"), TensorSpec(name + ".b", (width,), VECTOR)]
+        specs = [TensorSpec(name, (width,), VECTOR, "one_plus_normal")]
+        if spec.params.get("bias", True):
+            specs.append(TensorSpec(name + ".b", (width,), VECTOR))
+        return specs
 
     @classmethod
     def check_supported(cls, spec: PartSpec, dtype: torch.dtype) -> None:
@@ -104,7 +108,8 @@ class LayerNorm(Norm):
 
     def load(self, tensors: Dict[str, torch.Tensor]) -> None:
         name = f"{self.prefix}{self.spec.params['tensor']}"
-        self.weight, self.bias = tensors[name], tensors[name + ".b"]
+        self.weight = tensors[name]
+        self.bias = tensors[name + ".b"] if self.spec.params.get("bias", True) else None
 
     def as_kernel(self):
         return "layer", self.weight, self.bias, self.eps

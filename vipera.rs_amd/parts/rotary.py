@@ -118,6 +118,12 @@ class RotaryNeox(PositionEncoding):
                              batch.entry_of_token, None, heads, kv_heads, head_dim, self.step_angles(batch))
 
 
+def prompt_angles(position: PositionEncoding, batch, rotary_dim: int):
+    """The table of the step's sines and cosines where the step has enough tokens to share one, else None: the kernel then
+    computes them itself (with the position part's amplitude)."""
+    return position.step_angles(batch) if rotary_dim and batch.num_tokens >= ANGLE_TABLE_MIN_TOKENS else None
+
+
 class NoPosition(PositionEncoding):
     """No position encoding: queries and keys stay as projected."""
 
