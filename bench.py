@@ -92,7 +92,7 @@ def main() -> int:
                         help="also run one decode step (of --batch requests at --ctx) and one prefill eagerly with a "
                              "pair of GPU events around every kernel launch, and add the microseconds of each class of "
                              "kernel to the line (split_decode_us, split_prefill_us)")
-    parser.add_argument("--design", default="", choices=["", "gilidra", "zulesun", "muzasun", "lurirax", "zeladra"],
+    parser.add_argument("--design", default="", choices=["", "gilidra", "zulesun", "muzasun", "lurirax", "zeladra", "rebidra"],
                         help="instead of the headline measurement: prefill and decode of this design at layer sizes that "
                              "resemble a real model's (--size), beside the dense Qwen2 decoder of the same width, depth and "
                              "active feed-forward width, each with the time of every class of kernel")
@@ -487,6 +487,22 @@ def zeladra_shape(z):
             "embedding": {"scale": 1.0}, "layers": layers}
 
 
+def rebidra_shape(z):
+    """A Rebidra configuration of sizes ``z``: attention in a sliding window with a sink in every layer, convolutions of four
+    taps, values that are the keys, a mixture of ungated experts with a gated shared one, a side table of 64 columns a layer;
+    three layers fewer than ``z`` names, of which three run twice, so that a token passes as many layers."""
+    heads = z["heads"]
+    moe = {"kind": "moe", "expert": {"ff": z["ff"]}, "router": {"experts": z["experts"], "top": z["top"]},
+           "shared": {"ff": z["ff"]}}
+    window = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": z["dim"], "vdim": z["dim"], "conv": 4,
+              "mask": {"size": z["window"]}, "scale": z["dim"] ** -0.5,
+              "rot": {"base": 1e6, "dims": z["dim"], "scaling": {"factor": 8.0, "fast": 32.0, "slow": 1.0, "original": 8192}}}
+    layers = [{"type": "attention", "mixer": window, "mlp": moe} for _ in range(z["layers"] - 3)]
+    return {"architecture": "Rebidra", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-5}, "logit_scale": 0.5,
+            "embedding": {"scale": 1.0}, "token_side": {"dim": 64}, "loop": {"start": 2, "stop": 5, "times": 2},
+            "layers": layers}
+
+
 def dense_shape(z):
     """The dense Qwen2 decoder of the same width, depth, heads and active feed-forward width."""
     return dict(QWEN25_7B, num_hidden_layers=z["layers"], hidden_size=z["width"], num_attention_heads=z["heads"],
@@ -517,16 +533,14 @@ def design_comparison(args) -> int:
     out = {}
     # Gilidra beside the dense decoder; Zulesun and Muzasun each beside Gilidra, the engine's other decoder of
     # recurrences and mixtures of experts behind Dynamic Tanh norms, and beside the dense decoder; Zeladra beside Gilidra
-    # (latent attention) and Zulesun (a scan behind a convolution) and beside the dense decoder
-    runs = ((("gilidra", gilidra_shape(z)), ("dense", dense_shape(z))) if args.design == "gilidra" else
-            (("muzasun", muzasun_shape(z)), ("gilidra", gilidra_shape(z)), ("dense", dense_shape(z)))
-            if args.design == "muzasun" else
-            (("lurirax", lurirax_shape(z)), ("zulesun", zulesun_shape(z)), ("dense", dense_shape(z)))
-            if args.design == "lurirax" else
-            (("zeladra", zeladra_shape(z)), ("gilidra", gilidra_shape(z)), ("zulesun", zulesun_shape(z)),
-             ("dense", dense_shape(z))) if args.design == "zeladra" else
-            (("zulesun", zulesun_shape(z)), ("gilidra", gilidra_shape(z)), ("dense", dense_shape(z))))
-    for name, shape in runs:
+    # (latent attention) and Zulesun (a scan behind a convolution) and beside the dense decoder; Rebidra beside Lurirax
+    # (windows with a sink, experts with a gated shared one) and Zulesun (a side table) and beside the dense decoder
+    shapes = {"gilidra": gilidra_shape, "zulesun": zulesun_shape, "muzasun": muzasun_shape, "lurirax": lurirax_shape,
+              "zeladra": zeladra_shape, "rebidra": rebidra_shape, "dense": dense_shape}
+    beside = {"gilidra": [], "zulesun": ["gilidra"], "muzasun": ["gilidra"], "lurirax": ["zulesun"],
+              "zeladra": ["gilidra", "zulesun"], "rebidra": ["lurirax", "zulesun"]}[args.design]
+    for name in [args.design, *beside, "dense"]:
+        shape = shapes[name](z)
         config = config_from_dict(shape)
         runtime = Runtime("cuda:0", args.dtype)
         model = build_model(config, runtime)
@@ -587,10 +601,8 @@ def design_comparison(args) -> int:
         out[name] = result
         del runner, model
         torch.cuda.empty_cache()
-    print(json.dumps({"metric": f"prefill and decode of {args.design} beside " + ("the dense decoder" if args.design == "gilidra"
-                                                                                    else "Zulesun and the dense decoder" if args.design == "lurirax"
-                                                                                    else "Gilidra, Zulesun and the dense decoder" if args.design == "zeladra"
-                                                                                    else "Gilidra and the dense decoder") + " of equal size",
+    others = " and ".join(part for part in (", ".join(other.capitalize() for other in beside), "the dense decoder") if part)
+    print(json.dumps({"metric": f"prefill and decode of {args.design} beside {others} of equal size",
                       "size": z, "dtype": args.dtype, "prefill_tokens": T, "ctx": ctx, "data": "synthetic: seeded random "
                       "weights and uniform-random token ids", **out}), flush=True)
     return 0
