@@ -522,7 +522,7 @@ __global__ __launch_bounds__(PT_THREADS) void attn_prefill_kernel(
   l = sum_of_column(l);
   if (!col_ok) return;
   if (ex.sink) l += __builtin_amdgcn_exp2f(__builtin_fmaf(ex.sink[h], 1.44269504088896341f, -m * c2));   // m is a raw score
-  const float inv = 1.f / l;
+  const float inv = output_gate(ex, tok0 + c, h) / l;
   __bf16* dst = out + (size_t)(tok0 + c) * heads * hd + (size_t)h * hd;
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt) {
@@ -852,7 +852,7 @@ __global__ __launch_bounds__(SPLIT ? 2 * PT_THREADS : PT_THREADS) void attn_pref
     return;
   }
   if (ex.sink) l += __builtin_amdgcn_exp2f(__builtin_fmaf(ex.sink[h], 1.44269504088896341f, -m * c2));   // m is a raw score
-  const float inv = 1.f / l;
+  const float inv = output_gate(ex, tok0 + c, h) / l;
   __bf16* dst = out + (size_t)(tok0 + c) * heads * hd + (size_t)h * hd;
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt) {
@@ -915,7 +915,7 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(const float* __
       }
   }
   if (ex.sink) total += __builtin_amdgcn_exp2f(__builtin_fmaf(ex.sink[h], 1.44269504088896341f, -best * c2));
-  const float inv = 1.f / total;
+  const float inv = output_gate(ex, tok0 + tile_off + col, h) / total;
   bf16x4 r;
 #pragma unroll
   for (int j = 0; j < 4; ++j) r[j] = (__bf16)(acc[j] * inv);
@@ -1020,7 +1020,7 @@ __global__ __launch_bounds__(JOINED ? JOINED_WAVES * 64 : 64) __attribute__((amd
       total += (mc > -INFINITY ? __expf(mc - best) : 0.f) * max_sum[(c * 16 + lr) * 2 + 1];
     }
     if (EXT && ex.sink && col_ok) total += __expf(ex.sink[h] - best);
-    const float inv = 1.f / total;
+    const float inv = (EXT && col_ok ? output_gate(ex, token, h) : 1.f) / total;
     for (int dt = wave; dt < DT; dt += chunks) {
       f32x4 acc = {0.f, 0.f, 0.f, 0.f};
       for (int c = 0; c < chunks; ++c) {
@@ -1062,7 +1062,7 @@ __global__ __launch_bounds__(CB_THREADS) void attn_combine_kernel(const float* _
                                                                   __bf16* __restrict__ out,
                                                                   const int* __restrict__ entries,
                                                                   const int* __restrict__ entry_start, int heads, int hd,
-                                                                  int chunks, const float* __restrict__ sink) {
+                                                                  int chunks, AttnExtras ex) {
   __shared__ float weight[MAX_CHUNKS];
   __shared__ float wave_best[4], wave_total[4];
   __shared__ f32x4 part_sum[CB_THREADS];
@@ -1075,6 +1075,7 @@ __global__ __launch_bounds__(CB_THREADS) void attn_combine_kernel(const float* _
   const bool active = part < parts;
   constexpr int AHEAD = 4;
   const int token = entry_start[entries[slot]];
+  const float gate = output_gate(ex, token, h);
   f32x4 ahead[AHEAD];
 #pragma unroll
   for (int u = 0; u < AHEAD; ++u) {
@@ -1093,8 +1094,8 @@ __global__ __launch_bounds__(CB_THREADS) void attn_combine_kernel(const float* _
   const float mine = wave_sum(w * lc);
   if (lane == 0) wave_total[wave] = mine;
   __syncthreads();
-  const float inv = 1.f / ((((wave_total[0] + wave_total[1]) + wave_total[2]) + wave_total[3])
-                           + (sink ? __expf(sink[h] - best) : 0.f));
+  const float inv = gate / ((((wave_total[0] + wave_total[1]) + wave_total[2]) + wave_total[3])
+                           + (ex.sink ? __expf(ex.sink[h] - best) : 0.f));
   f32x4 acc = {0.f, 0.f, 0.f, 0.f};
   if (active) {
     int c = part;
@@ -1134,15 +1135,15 @@ extern "C" int vk_attn_bf16_hdp() { return HDP; }
 // chunk_tiles > 0 (with the kernel that loads straight into LDS; ignored otherwise): a tile's steps of 64 positions
 // are cut into chunks of that many, a workgroup each, of which no tile has more than `max_chunks`; `partial` holds
 // num_tiles * heads * max_chunks * 128 * (padded head width + 4) floats.
-// sink, rel, rel_far, keep_first: see attn_extras.h (null, null, 0, 0: none of them).
+// sink, rel, rel_far, keep_first, gate, gate_ld: see attn_extras.h (null and 0: none of them).
 extern "C" int vk_attn_bf16_prefill_ext(const void* q, long long q_stride, const void* k_cache, const void* v_cache,
                                     void* out, const int* tiles, int num_tiles, const int* entry_start,
                                     const int* entry_first_pos, const int* block_table, int table_width,
                                     int block_size, int heads, int kv_heads, int hd, float scale, int window, float softcap,
                                     int split, float* partial, long long partial_floats, int chunk_tiles,
                                     int max_chunks, const float* sink, const float* rel, int rel_far, int keep_first,
-                                    void* stream) {
-  const AttnExtras ex{sink, rel, rel_far, keep_first};
+                                    const float* gate, long long gate_ld, void* stream) {
+  const AttnExtras ex{sink, rel, rel_far, keep_first, gate, gate_ld};
   if (rel_far < 0 || keep_first < 0 || (keep_first > 0 && window <= 0)) return VK_BAD_ARGUMENT;
   if (num_tiles <= 0) return 0;
   if (hd <= 0 || hd > HDP || (hd & 7) || block_size <= 0 || (block_size & 7) || heads <= 0 || kv_heads <= 0 ||
@@ -1226,7 +1227,7 @@ extern "C" int vk_attn_bf16_prefill_capped(const void* q, long long q_stride, co
                                     int max_chunks, void* stream) {
   return vk_attn_bf16_prefill_ext(q, q_stride, k_cache, v_cache, out, tiles, num_tiles, entry_start, entry_first_pos,
                                   block_table, table_width, block_size, heads, kv_heads, hd, scale, window, softcap, split,
-                                  partial, partial_floats, chunk_tiles, max_chunks, nullptr, nullptr, 0, 0, stream);
+                                  partial, partial_floats, chunk_tiles, max_chunks, nullptr, nullptr, 0, 0, nullptr, 0, stream);
 }
 
 // entries: indices of the step's entries that hold exactly one token. partial: at least
@@ -1238,8 +1239,9 @@ extern "C" int vk_attn_bf16_decode_ext(const void* q, long long q_stride, const 
                                    const int* entry_start, const int* entry_first_pos, const int* block_table,
                                    int table_width, int block_size, int heads, int kv_heads, int hd, float scale,
                                    int window, float softcap, int chunk, int chunks, int dense, int join,
-                                   const float* sink, const float* rel, int rel_far, int keep_first, void* stream) {
-  const AttnExtras ex{sink, rel, rel_far, keep_first};
+                                   const float* sink, const float* rel, int rel_far, int keep_first,
+                                   const float* gate, long long gate_ld, void* stream) {
+  const AttnExtras ex{sink, rel, rel_far, keep_first, gate, gate_ld};
   if (rel_far < 0 || keep_first < 0 || (keep_first > 0 && window <= 0)) return VK_BAD_ARGUMENT;
   if (num_entries <= 0) return 0;
   if (hd <= 0 || hd > HDP || (hd & 7) || block_size <= 0 || (block_size & 7) || heads <= 0 || kv_heads <= 0 ||
@@ -1251,7 +1253,7 @@ extern "C" int vk_attn_bf16_decode_ext(const void* q, long long q_stride, const 
   const int group = heads / kv_heads, head_blocks = (group + 15) / 16;
   if (kv_heads * head_blocks > 65535 || heads > 65535) return VK_UNSUPPORTED_SIZE;
   hipStream_t s = (hipStream_t)stream;
-  const bool ext = softcap > 0.f || window < 0 || sink || rel || keep_first > 0;
+  const bool ext = softcap > 0.f || window < 0 || sink || rel || keep_first > 0 || gate;
   // pages a chunk can touch: chunks start at multiples of `chunk`, which need not be page edges
   const int chunk_pages = chunk % block_size == 0 ? chunk / block_size : chunk / block_size + 2;
   if (join) {
@@ -1281,7 +1283,7 @@ extern "C" int vk_attn_bf16_decode_ext(const void* q, long long q_stride, const 
                              heads, kv_heads, hd, scale, window, softcap, chunk, head_blocks, dense, ex);
   VK_LAUNCH_CHECK();
   dim3 cgrid(num_entries, heads);
-  attn_combine_kernel<<<cgrid, CB_THREADS, 0, s>>>(partial, (__bf16*)out, entries, entry_start, heads, hd, chunks, sink);
+  attn_combine_kernel<<<cgrid, CB_THREADS, 0, s>>>(partial, (__bf16*)out, entries, entry_start, heads, hd, chunks, ex);
   VK_LAUNCH_CHECK();
   return 0;
 }
@@ -1293,7 +1295,7 @@ extern "C" int vk_attn_bf16_decode_capped(const void* q, long long q_stride, con
                                    int window, float softcap, int chunk, int chunks, int dense, int join, void* stream) {
   return vk_attn_bf16_decode_ext(q, q_stride, k_cache, v_cache, out, partial, entries, num_entries, entry_start,
                                  entry_first_pos, block_table, table_width, block_size, heads, kv_heads, hd, scale, window,
-                                 softcap, chunk, chunks, dense, join, nullptr, nullptr, 0, 0, stream);
+                                 softcap, chunk, chunks, dense, join, nullptr, nullptr, 0, 0, nullptr, 0, stream);
 }
 
 // The same two without a cap on the scores.

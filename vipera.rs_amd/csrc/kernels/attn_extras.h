@@ -3,6 +3,7 @@
 //   rel, rel_far  [heads, rel_far + 1] 32-bit: rel[h, min(i - j, rel_far)] is added to the scaled score of query
 //               position i and key position j (a table by distance, made by the host from whatever the model learned)
 //   keep_first  with a window: positions below keep_first stay visible whatever the window has passed
+//   gate, gate_ld  [tokens, gate_ld] 32-bit: head h's output of token t is multiplied by sigmoid(gate[t * gate_ld + h])
 #pragma once
 #include "common.h"
 
@@ -11,7 +12,14 @@ struct AttnExtras {
   const float* rel;
   int rel_far;
   int keep_first;
+  const float* gate;
+  long long gate_ld;
 };
+
+// What a head's output of a token is multiplied by.
+__device__ __forceinline__ float output_gate(const AttnExtras& x, int token, int head) {
+  return x.gate ? 1.0f / (1.0f + expf(-x.gate[token * x.gate_ld + head])) : 1.f;
+}
 
 // Whether the token at `pos` sees position p, for p <= pos.
 __device__ __forceinline__ bool sees_position(int p, int pos, int window, int keep_first) {

@@ -96,7 +96,7 @@ __global__ __launch_bounds__(THREADS) void attn_generic_kernel(
   if (tid < hd) {
     float total = 0.f;
     for (int pidx = 0; pidx < parts; ++pidx) total += part_s[pidx * hd + tid];
-    out[(size_t)t * heads * hd + (size_t)h * hd + tid] = from_float<T>(total / (l + sink_term(ex, h, m)));
+    out[(size_t)t * heads * hd + (size_t)h * hd + tid] = from_float<T>(total / (l + sink_term(ex, h, m)) * output_gate(ex, t, h));
   }
 }
 
@@ -330,7 +330,7 @@ __global__ __launch_bounds__(64) void attn_combine_f32_kernel(const float* __res
         sum = fmaf(src[(size_t)ch * stride + hd + 1], factor, sum);
       }
     }
-    out[(size_t)token * heads * hd + (size_t)h * hd + d] = from_float<T>(total / (sum + sink_term(ex, h, best)));
+    out[(size_t)token * heads * hd + (size_t)h * hd + d] = from_float<T>(total / (sum + sink_term(ex, h, best)) * output_gate(ex, token, h));
   }
 }
 
@@ -514,9 +514,9 @@ __global__ __launch_bounds__(256) void attn_prefill_f32_kernel(
   for (int i = 0; i < 4; ++i) {
     if (4 * ty + i >= rows) continue;
     float* dst = out + (size_t)(tok0 + 4 * ty + i) * heads * HD + (size_t)h * HD;
-    const float whole = l[i] + sink_term(ex, h, m[i]);
+    const float whole = l[i] + sink_term(ex, h, m[i]), gate = output_gate(ex, tok0 + 4 * ty + i, h);
 #pragma unroll
-    for (int j = 0; j < DPT; ++j) dst[tx + 16 * j] = o[i][j] / whole;
+    for (int j = 0; j < DPT; ++j) dst[tx + 16 * j] = o[i][j] / whole * gate;
   }
 }
 
@@ -560,8 +560,9 @@ extern "C" int vk_attn_generic_ext(const void* q, long long q_stride, const void
                                void* out, int dtype, const int* positions, const int* entry_of_token,
                                const int* block_table, int table_width, int block_size, int num_tokens, int heads,
                                int kv_heads, int hd, float scale, int window, float softcap, const int* skip_single_of,
-                               const float* sink, const float* rel, int rel_far, int keep_first, void* stream) {
-  const AttnExtras ex{sink, rel, rel_far, keep_first};
+                               const float* sink, const float* rel, int rel_far, int keep_first, const float* gate, long long gate_ld,
+                               void* stream) {
+  const AttnExtras ex{sink, rel, rel_far, keep_first, gate, gate_ld};
   if (!extras_ok(ex, window)) return VK_BAD_ARGUMENT;
   if (num_tokens <= 0) return 0;
   if (hd <= 0 || hd > MAX_HD) return VK_UNSUPPORTED_SIZE;
@@ -592,7 +593,7 @@ extern "C" int vk_attn_generic_capped(const void* q, long long q_stride, const v
                                void* stream) {
   return vk_attn_generic_ext(q, q_stride, k_cache, v_cache, out, dtype, positions, entry_of_token, block_table,
                              table_width, block_size, num_tokens, heads, kv_heads, hd, scale, window, softcap,
-                             skip_single_of, nullptr, nullptr, 0, 0, stream);
+                             skip_single_of, nullptr, nullptr, 0, 0, nullptr, 0, stream);
 }
 
 
@@ -606,8 +607,9 @@ extern "C" int vk_attn_decode_f32_ext(const float* q, long long q_stride, const 
                                   const int* entry_start, const int* entry_first_pos, const int* block_table,
                                   int table_width, int block_size, int heads, int kv_heads, int hd, float scale,
                                   int window, float softcap, int chunks, const float* sink, const float* rel, int rel_far,
-                                  int keep_first, void* stream) {
-  const AttnExtras ex{sink, rel, rel_far, keep_first};
+                                  int keep_first, const float* gate, long long gate_ld,
+                               void* stream) {
+  const AttnExtras ex{sink, rel, rel_far, keep_first, gate, gate_ld};
   if (!extras_ok(ex, window)) return VK_BAD_ARGUMENT;
   if (num_entries <= 0) return 0;
   if (hd <= 0 || hd > MAX_HD || (hd & 3) || block_size <= 0 || (block_size & 3) || (q_stride & 3)) return VK_UNSUPPORTED_SIZE;
@@ -649,7 +651,7 @@ extern "C" int vk_attn_decode_f32_capped(const float* q, long long q_stride, con
                                   int window, float softcap, int chunks, void* stream) {
   return vk_attn_decode_f32_ext(q, q_stride, k_cache, v_cache, out, partial, entries, num_entries, entry_start,
                                 entry_first_pos, block_table, table_width, block_size, heads, kv_heads, hd, scale, window,
-                                softcap, chunks, nullptr, nullptr, 0, 0, stream);
+                                softcap, chunks, nullptr, nullptr, 0, 0, nullptr, 0, stream);
 }
 
 // Attention of the step's prompt portions in 32-bit: float q, cache and out. tiles: pairs (entry, first token of the
@@ -659,8 +661,9 @@ extern "C" int vk_attn_prefill_f32_ext(const float* q, long long q_stride, const
                                    float* out, const int* tiles, int num_tiles, int tile_tokens, const int* entry_start,
                                    const int* entry_first_pos, const int* block_table, int table_width, int block_size,
                                    int heads, int kv_heads, int hd, float scale, int window, float softcap,
-                                   const float* sink, const float* rel, int rel_far, int keep_first, void* stream) {
-  const AttnExtras ex{sink, rel, rel_far, keep_first};
+                                   const float* sink, const float* rel, int rel_far, int keep_first, const float* gate, long long gate_ld,
+                               void* stream) {
+  const AttnExtras ex{sink, rel, rel_far, keep_first, gate, gate_ld};
   if (!extras_ok(ex, window)) return VK_BAD_ARGUMENT;
   if (num_tiles <= 0) return 0;
   if (hd <= 0 || hd > 128 || (hd & 15) || block_size <= 0 || (block_size & 3) || (q_stride & 3)) return VK_UNSUPPORTED_SIZE;
@@ -691,7 +694,7 @@ extern "C" int vk_attn_prefill_f32_capped(const float* q, long long q_stride, co
                                    int heads, int kv_heads, int hd, float scale, int window, float softcap, void* stream) {
   return vk_attn_prefill_f32_ext(q, q_stride, k_cache, v_cache, out, tiles, num_tiles, tile_tokens, entry_start,
                                  entry_first_pos, block_table, table_width, block_size, heads, kv_heads, hd, scale, window,
-                                 softcap, nullptr, nullptr, 0, 0, stream);
+                                 softcap, nullptr, nullptr, 0, 0, nullptr, 0, stream);
 }
 
 // The same three without a cap on the scores.

@@ -185,188 +185,200 @@ template <typename TO> struct ConvHeads {
 
 template <typename TO, int R, int K, int TW>
 __global__ __launch_bounds__(256) void head_conv_prepare_kernel(ConvHeads<TO> a, long long units) {
-  __shared__ float turned[4][R * WAVE];
+  __shared__ float turned[4][TW][R * WAVE];
   const int lane = threadIdx.x & (WAVE - 1), wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
   const long long unit = (long long)blockIdx.x * (blockDim.x / WAVE) + wave;
   if (unit >= units) return;                             // a wave's work is its own: no barrier follows
   const int qk = a.heads + a.kv_heads, per_token = qk + (a.own_values ? a.kv_heads : 0);
   const int u = (int)(unit % per_token);
-  const int t0 = (int)(unit / per_token) * TW, t1 = min(t0 + TW, a.tokens);
+  const int t0 = (int)(unit / per_token) * TW, count = min(TW, a.tokens - t0);
   const bool is_q = u < a.heads, is_v = u >= qk;
   const int g = is_q ? 0 : is_v ? u - qk : u - a.heads;
   const int n = is_v ? a.vdim : a.dim;
   const long long base = is_v ? (long long)qk * a.dim + (long long)g * a.vdim : (long long)u * a.dim;
   const int C = qk * a.dim, taps = is_v || !a.conv ? 1 : a.taps;
-  const bool gives_values = is_v || (!is_q && !a.own_values);
   constexpr int P = K > 1 ? K - 1 : 1;
-  float w[K > 0 ? K : 1][R], past[P][R], x[TW][R], norm_weight[R];
+  // everything the run needs is asked for before anything is used; a token past the step's last repeats it
+  int entry[TW], pos[TW];
+  float x[TW][R], w[K > 0 ? K : 1][R], norm_weight[R];
   const float* weight = is_q ? a.q_weight : a.k_weight;
+#pragma unroll
+  for (int i = 0; i < TW; ++i) {
+    const int t = min(t0 + i, a.tokens - 1);
+    entry[i] = a.entry_of[t];
+    pos[i] = a.positions[t];
+#pragma unroll
+    for (int r = 0; r < R; ++r) x[i][r] = lane + WAVE * r < n ? a.proj[(long long)t * a.ldp + base + lane + WAVE * r] : 0.f;
+  }
 #pragma unroll
   for (int r = 0; r < R; ++r) {
     const int d = lane + WAVE * r;
     const bool in = d < n;
-#pragma unroll
-    for (int i = 0; i < TW; ++i) x[i][r] = in ? a.proj[(long long)min(t0 + i, a.tokens - 1) * a.ldp + base + d] : 0.f;
     if constexpr (K > 0) {
 #pragma unroll
       for (int j = 0; j < K; ++j) {
         const int at = j - (K - taps);                   // column of the stored taps
-        w[j][r] = !in || at < 0 ? 0.f : taps > 1 || (a.conv && !is_v) ? a.conv[(base + d) * taps + at] : 1.f;
+        w[j][r] = !in || at < 0 ? 0.f : a.conv && !is_v ? a.conv[(base + d) * taps + at] : 1.f;
       }
     }
     norm_weight[r] = (in && a.norm && weight && !is_v) ? weight[d] : 1.f;
   }
-  TO held[TW][R];
-  int of = -1, run_entry = -1, run_first = 0;
+  int page[TW];
 #pragma unroll
-  for (int i = 0; i < TW; ++i) {
-    const int t = t0 + i;
-    if (t >= t1) break;
-    const int e = a.entry_of[t], pos = a.positions[t];
-    const int offset = t - a.entry_start[e];
-    const bool fresh = a.entry_first[e] == 0;
-    float* old = a.conv ? a.state + (long long)a.slots[e] * a.state_stride + base : nullptr;
-    // a channel's input `back` tokens before t; `back` is at least 1 and below taps
-    auto before = [&](int back, int d) -> float {
-      if (back <= offset) return a.proj[(long long)(t - back) * a.ldp + base + d];
-      return fresh ? 0.f : old[(long long)(taps - 1 - (back - offset)) * C + d];
-    };
-    float y[R];
-    if constexpr (K > 0) {
-      if (e != of) {                                     // the run's first token, or another entry's
-        of = e;
+  for (int i = 0; i < TW; ++i) page[i] = is_q ? -1 : a.table[(size_t)entry[i] * a.table_width + pos[i] / a.block_size];
+  // a channel's input `back` tokens before token i of the run; `back` is at least 1 and below taps
+  auto before = [&](int i, int back, int d) -> float {
+    const int e = entry[i], t = min(t0 + i, a.tokens - 1), offset = t - a.entry_start[e];
+    if (back <= offset) return a.proj[(long long)(t - back) * a.ldp + base + d];
+    return a.entry_first[e] == 0 ? 0.f : a.state[(long long)a.slots[e] * a.state_stride + base + (long long)(taps - 1 - (back - offset)) * C + d];
+  };
+  float y[TW][R];
+  if constexpr (K > 0) {
+    float past[P][R];
+#pragma unroll
+    for (int i = 0; i < TW; ++i) {
+      if (i == 0 || entry[i] != entry[i > 0 ? i - 1 : 0]) {        // the run's first token, or another entry's
 #pragma unroll
         for (int j = 0; j < K - 1; ++j)
 #pragma unroll
           for (int r = 0; r < R; ++r) {
             const int d = lane + WAVE * r, back = K - 1 - j;
-            past[j][r] = (d < n && back < taps) ? before(back, d) : 0.f;
+            past[j][r] = (d < n && back < taps) ? before(i, back, d) : 0.f;
           }
+      }
+      if (TW == 1 && a.keep && taps > 1) {
+        // row j of the state becomes the input taps - 2 - j tokens before this one
+        float* old = a.state + (long long)a.slots[entry[i]] * a.state_stride + base;
+#pragma unroll
+        for (int r = 0; r < R; ++r)
+#pragma unroll
+          for (int back = 0; back < K - 1; ++back)
+            if (lane + WAVE * r < n && back < taps - 1)
+              old[(long long)(taps - 2 - back) * C + lane + WAVE * r] = back ? past[K - 1 - back][r] : x[i][r];
       }
 #pragma unroll
       for (int r = 0; r < R; ++r) {
         float sum = 0.f;
 #pragma unroll
         for (int j = 0; j < K - 1; ++j) sum = fmaf(w[j][r], past[j][r], sum);
-        y[r] = fmaf(w[K - 1][r], x[i][r], sum);
-        if (TW == 1 && a.keep && taps > 1 && lane + WAVE * r < n) {
-          // row j of the state becomes the input taps - 2 - j tokens before this one
-#pragma unroll
-          for (int back = 0; back < K - 1; ++back)
-            if (back < taps - 1) old[(long long)(taps - 2 - back) * C + lane + WAVE * r] = back ? past[K - 1 - back][r] : x[i][r];
-        }
+        y[i][r] = fmaf(w[K - 1][r], x[i][r], sum);
 #pragma unroll
         for (int j = 0; j + 1 < K - 1; ++j) past[j][r] = past[j + 1][r];
         past[P - 1][r] = x[i][r];
       }
-    } else {
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < TW; ++i) {
+      float* old = a.state + (long long)a.slots[entry[i]] * a.state_stride + base;
 #pragma unroll
       for (int r = 0; r < R; ++r) {
         const int d = lane + WAVE * r;
-        y[r] = 0.f;
+        y[i][r] = 0.f;
         if (d >= n) continue;
         float sum = 0.f;
         for (int j = 0; j + 1 < taps; ++j) {
-          const float v = before(taps - 1 - j, d);
+          const float v = before(i, taps - 1 - j, d);
           sum = fmaf(a.conv[(base + d) * taps + j], v, sum);
           if (TW == 1 && a.keep && j > 0) old[(long long)(j - 1) * C + d] = v;
         }
-        y[r] = taps > 1 || (a.conv && !is_v) ? fmaf(a.conv[(base + d) * taps + taps - 1], x[i][r], sum) : x[i][r];
+        y[i][r] = taps > 1 ? fmaf(a.conv[(base + d) * taps + taps - 1], x[i][r], sum) : x[i][r];
         if (TW == 1 && a.keep && taps > 1) old[(long long)(taps - 2) * C + d] = x[i][r];
       }
     }
-    if (i == 0) {
-      run_entry = e;
-      run_first = pos;
-    } else if (e != run_entry) {
-      run_entry = -1;
-    }
-    const int page = is_q ? -1 : a.table[(size_t)e * a.table_width + pos / a.block_size], slot = pos % a.block_size;
-    if (gives_values) {
+  }
+  if (is_v || (!is_q && !a.own_values)) {
+    // the run's values, transposed: consecutive positions of a number lie side by side in its page
+    constexpr int PIECE = 16 / (int)sizeof(TO);
+    bool whole = TW % PIECE == 0 && count == TW && pos[0] % TW == 0 && a.block_size % TW == 0 && page[0] >= 0;
 #pragma unroll
-      for (int r = 0; r < R; ++r) held[i][r] = from_float<TO>(lane + WAVE * r < n ? y[r] : 0.f);
-    }
-    if (is_v) continue;
-    if (a.norm) {
-      float ss = 0.f;
-#pragma unroll
-      for (int r = 0; r < R; ++r) ss = fmaf(y[r], y[r], ss);
-      const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)n + a.eps);
-#pragma unroll
-      for (int r = 0; r < R; ++r) y[r] = y[r] * inv * norm_weight[r];
-    }
-    if (a.rot_dims > 0) {
-      const int half = a.rot_dims / 2;
-#pragma unroll
-      for (int r = 0; r < R; ++r) turned[wave][lane + WAVE * r] = y[r];
-      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-      __builtin_amdgcn_wave_barrier();
+    for (int i = 1; i < TW; ++i) whole = whole && entry[i] == entry[0];
+    if (whole) {
+      typedef TO piece_t __attribute__((ext_vector_type(PIECE)));
 #pragma unroll
       for (int r = 0; r < R; ++r) {
         const int d = lane + WAVE * r;
-        if (d >= a.rot_dims) continue;
-        const int pair = d < half ? d : d - half;
-        const float other = turned[wave][d < half ? d + half : d - half];
+        if (d >= a.W) continue;
+        TO* dst = a.v_cache + (((size_t)page[0] * a.kv_heads + g) * a.W + d) * a.block_size + pos[0] % a.block_size;
+#pragma unroll
+        for (int p = 0; p < TW / PIECE; ++p) {
+          piece_t v;
+#pragma unroll
+          for (int i = 0; i < PIECE; ++i) v[i] = from_float<TO>(y[(p * PIECE + i) % TW][r]);
+          *(piece_t*)(dst + p * PIECE) = v;
+        }
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < TW; ++i) {
+        if (i >= count || page[i] < 0) continue;
+        TO* dst = a.v_cache + ((size_t)page[i] * a.kv_heads + g) * a.W * a.block_size + pos[i] % a.block_size;
+#pragma unroll
+        for (int r = 0; r < R; ++r)
+          if (lane + WAVE * r < a.W) dst[(size_t)(lane + WAVE * r) * a.block_size] = from_float<TO>(y[i][r]);
+      }
+    }
+    if (is_v) return;
+  }
+  if (a.norm) {
+    float ss[TW];
+#pragma unroll
+    for (int i = 0; i < TW; ++i) {
+      ss[i] = 0.f;
+#pragma unroll
+      for (int r = 0; r < R; ++r) ss[i] = fmaf(y[i][r], y[i][r], ss[i]);
+    }
+#pragma unroll
+    for (int off = WAVE / 2; off > 0; off >>= 1)         // the tokens' sums step by step side by side
+#pragma unroll
+      for (int i = 0; i < TW; ++i) ss[i] += __shfl_xor(ss[i], off, WAVE);
+#pragma unroll
+    for (int i = 0; i < TW; ++i) {
+      const float inv = 1.0f / sqrtf(ss[i] / (float)n + a.eps);
+#pragma unroll
+      for (int r = 0; r < R; ++r) y[i][r] = y[i][r] * inv * norm_weight[r];
+    }
+  }
+  if (a.rot_dims > 0) {
+    const int half = a.rot_dims / 2;
+#pragma unroll
+    for (int i = 0; i < TW; ++i)
+#pragma unroll
+      for (int r = 0; r < R; ++r) turned[wave][i][lane + WAVE * r] = y[i][r];
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const int d = lane + WAVE * r;
+      if (d >= a.rot_dims) continue;
+      const int pair = d < half ? d : d - half;
+      const float sign = d < half ? -1.f : 1.f;
+      const float freq = a.angles ? 0.f : a.inv_freq[pair];
+#pragma unroll
+      for (int i = 0; i < TW; ++i) {
+        const float other = turned[wave][i][d < half ? d + half : d - half];
         float sn, cs;
         if (a.angles) {
-          const float2 v = a.angles[(long long)t * half + pair];
+          const float2 v = a.angles[(long long)min(t0 + i, a.tokens - 1) * half + pair];
           sn = v.x;
           cs = v.y;
         } else {
-          sincosf((float)pos * a.inv_freq[pair], &sn, &cs);
+          sincosf((float)pos[i] * freq, &sn, &cs);
           sn *= a.amplitude;
           cs *= a.amplitude;
         }
-        y[r] = d < half ? y[r] * cs - other * sn : y[r] * cs + other * sn;
-      }
-      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-      __builtin_amdgcn_wave_barrier();
-    }
-    if (!is_q && page < 0) continue;
-    TO* dst = is_q ? a.q + ((long long)t * a.heads + u) * a.W
-                   : a.k_cache + (((size_t)page * a.kv_heads + g) * a.block_size + slot) * a.W;
-#pragma unroll
-    for (int r = 0; r < R; ++r) {
-      const int d = lane + WAVE * r;
-      if (d < a.W) dst[d] = from_float<TO>(d < n ? y[r] : 0.f);
-    }
-  }
-  if (!gives_values) return;
-  // the run's values, transposed: consecutive positions of a number lie side by side in its page
-  constexpr int PIECE = 16 / (int)sizeof(TO);
-  const bool whole = TW % PIECE == 0 && t1 - t0 == TW && run_entry >= 0 && run_first % TW == 0 && a.block_size % TW == 0;
-  if (whole) {
-    const int page = a.table[(size_t)run_entry * a.table_width + run_first / a.block_size], slot = run_first % a.block_size;
-    if (page < 0) return;
-    typedef TO piece_t __attribute__((ext_vector_type(PIECE)));
-#pragma unroll
-    for (int r = 0; r < R; ++r) {
-      const int d = lane + WAVE * r;
-      if (d >= a.W) continue;
-      TO* dst = a.v_cache + (((size_t)page * a.kv_heads + g) * a.W + d) * a.block_size + slot;
-#pragma unroll
-      for (int p = 0; p < TW / PIECE; ++p) {
-        piece_t v;
-#pragma unroll
-        for (int i = 0; i < PIECE; ++i) v[i] = held[(p * PIECE + i) % TW][r];
-        *(piece_t*)(dst + p * PIECE) = v;
+        y[i][r] = y[i][r] * cs + sign * (other * sn);
       }
     }
-    return;
   }
 #pragma unroll
   for (int i = 0; i < TW; ++i) {
-    const int t = t0 + i;
-    if (t >= t1) break;
-    const int pos = a.positions[t];
-    const int page = a.table[(size_t)a.entry_of[t] * a.table_width + pos / a.block_size], slot = pos % a.block_size;
-    if (page < 0) continue;
-    TO* dst = a.v_cache + ((size_t)page * a.kv_heads + g) * a.W * a.block_size + slot;
+    if (i >= count || (!is_q && page[i] < 0)) continue;
+    TO* dst = is_q ? a.q + ((long long)(t0 + i) * a.heads + u) * a.W
+                   : a.k_cache + (((size_t)page[i] * a.kv_heads + g) * a.block_size + pos[i] % a.block_size) * a.W;
 #pragma unroll
-    for (int r = 0; r < R; ++r) {
-      const int d = lane + WAVE * r;
-      if (d < a.W) dst[(size_t)d * a.block_size] = held[i][r];
-    }
+    for (int r = 0; r < R; ++r)
+      if (lane + WAVE * r < a.W) dst[lane + WAVE * r] = from_float<TO>(y[i][r]);
   }
 }
 

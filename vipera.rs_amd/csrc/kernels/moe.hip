@@ -2,8 +2,8 @@
 //
 // A step's T tokens each choose `top` of E experts: P = T * top pairs, pair p = t * top + j.  The pairs are
 // grouped by expert (`order[i]` is the pair at sorted place i, `offsets[e]` the first place of expert e) and cut
-// into tiles of 64 places that never span two experts; a product's workgroup owns one tile and 64 output
-// columns.  The grid is sized for the most tiles there can be, and workgroups past `num_tiles` (which only the
+// into tiles of 64 places (128 on the matrix cores, 16 where a step has few pairs) that never span two experts; a
+// product's workgroup owns one tile and some output columns.  The grid is sized for the most tiles there can be, and workgroups past `num_tiles` (which only the
 // device knows) leave at once.  Which place a pair gets depends on the order in which the counters were bumped,
 // but no value does: a pair's row is computed alone, an FMA chain in k order per output element, and the
 // weighted sum over a token's choices runs in the order of the choices.
@@ -11,6 +11,7 @@
 #include "group_tile.h"
 
 constexpr int MOE_TILE = 64;      // places per tile of the 32-bit products; the matrix-core products take 128
+constexpr int MOE_FEW = 16;       // or 16, where the products are streams of the weights
 
 // ---------------------------------------------------------------------------------------------
 // One wave per token: the `top` largest of E logits (the lowest id wins a tie), and the softmax over those.
@@ -129,20 +130,35 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const float* __restrict
   __syncthreads();
   for (int p = threadIdx.x; p < pairs; p += blockDim.x) atomicAdd(&counts[ids[p]], 1);
   __syncthreads();
-  if (threadIdx.x == 0) {
+  if (threadIdx.x < WAVE) {          // one wave: running sums over the experts, 64 at a time
+    const int lane = threadIdx.x;
     int at = 0, tile = 0;
-    for (int e = 0; e < experts; ++e) {
-      offsets[e] = at;
-      cursor[e] = at;
-      for (int first = 0; first < counts[e]; first += tile_rows) {
-        tiles[2 * tile] = e;
-        tiles[2 * tile + 1] = at + first;
-        ++tile;
+    for (int base = 0; base < experts; base += WAVE) {
+      const int e = base + lane, count = e < experts ? counts[e] : 0, own = (count + tile_rows - 1) / tile_rows;
+      int places = count, tiles_upto = own;
+      for (int off = 1; off < WAVE; off <<= 1) {
+        const int p = __shfl_up(places, off, WAVE), q = __shfl_up(tiles_upto, off, WAVE);
+        if (lane >= off) {
+          places += p;
+          tiles_upto += q;
+        }
       }
-      at += counts[e];
+      if (e < experts) {
+        const int first = at + places - count;
+        offsets[e] = first;
+        cursor[e] = first;
+        for (int i = 0, to = tile + tiles_upto - own; i < own; ++i, ++to) {
+          tiles[2 * to] = e;
+          tiles[2 * to + 1] = first + i * tile_rows;
+        }
+      }
+      at += __shfl(places, WAVE - 1, WAVE);
+      tile += __shfl(tiles_upto, WAVE - 1, WAVE);
     }
-    offsets[experts] = at;
-    num_tiles[0] = tile;
+    if (lane == 0) {
+      offsets[experts] = at;
+      num_tiles[0] = tile;
+    }
   }
   __syncthreads();
   for (int p = threadIdx.x; p < pairs; p += blockDim.x) order[atomicAdd(&cursor[ids[p]], 1)] = p;
@@ -407,6 +423,92 @@ __global__ __launch_bounds__(256) void moe_down_mma_kernel(const __bf16* __restr
   }
 }
 
+// ---------------------------------------------------------------------------------------------
+// Few pairs an expert (decoding): the products are a stream of the chosen experts' weights.  A workgroup owns a tile of up to
+// 16 places and 32 weight rows (FORM 0, gate and up: the same 16 of either; 1, an up product without a gate; 2, down); its
+// four waves take a quarter of K each, straight from memory into v_mfma_f32_16x16x32_bf16 with the weight as the first
+// operand (a lane ends up with four consecutive outputs of one place), STREAM_STEPS steps of 32 k asked for ahead of the
+// ones that are multiplied, and add up through LDS in the order of the waves.
+constexpr int STREAM_STEPS = 4;
+template <int FORM>
+__global__ __launch_bounds__(256) void moe_stream_kernel(const __bf16* __restrict__ in, long long ldi,
+                                                         const __bf16* __restrict__ w0, const __bf16* __restrict__ w1,
+                                                         const int* __restrict__ offsets, const int* __restrict__ order,
+                                                         const int* __restrict__ tiles, const int* __restrict__ num_tiles,
+                                                         int top, int K, int N, float limit, float alpha, int plain,
+                                                         const float* __restrict__ in_weights, __bf16* __restrict__ act,
+                                                         float* __restrict__ pair_out) {
+  if ((int)blockIdx.y >= num_tiles[0]) return;
+  __shared__ gt_f32x4 part[4][2][WAVE];
+  const int e = tiles[2 * blockIdx.y], first = tiles[2 * blockIdx.y + 1];
+  const int count = min(MOE_FEW, offsets[e + 1] - first);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lr = lane & 15, lg = lane >> 4;
+  const int n0 = blockIdx.x * (FORM == 0 ? 16 : 32);
+  const long long matrix = (long long)e * N * K;
+  const __bf16* rows[2];
+#pragma unroll
+  for (int t = 0; t < 2; ++t) {
+    const int n = n0 + (FORM == 0 ? 0 : t * 16) + lr;
+    rows[t] = n < N ? ((FORM == 0 && t == 0) ? w0 : w1) + matrix + (long long)n * K : nullptr;
+  }
+  const __bf16* a_row = nullptr;
+  if (lr < count) a_row = in + (FORM == 2 ? (long long)(first + lr) : (long long)(order[first + lr] / top)) * ldi;
+  const int steps = (K + 31) / 32, quarter = (steps + 3) / 4;
+  const int s0 = wave * quarter, s1 = min(steps, s0 + quarter);
+  gt_f32x4 acc[2] = {gt_f32x4{0.f, 0.f, 0.f, 0.f}, gt_f32x4{0.f, 0.f, 0.f, 0.f}};
+  gt_bf16x8 fw[2][STREAM_STEPS][2], fa[2][STREAM_STEPS];
+  auto fetch = [&](int set, int s) {
+#pragma unroll
+    for (int i = 0; i < STREAM_STEPS; ++i) {
+      const int k = (s + i) * 32 + lg * 8;
+      const bool in_range = s + i < s1 && k < K;
+      gt_bf16x8 zero = {};
+#pragma unroll
+      for (int t = 0; t < 2; ++t) fw[set][i][t] = (rows[t] && in_range) ? *(const gt_bf16x8*)(rows[t] + k) : zero;
+      fa[set][i] = (a_row && in_range) ? *(const gt_bf16x8*)(a_row + k) : zero;
+    }
+  };
+  auto multiply = [&](int set) {
+#pragma unroll
+    for (int i = 0; i < STREAM_STEPS; ++i)
+#pragma unroll
+      for (int t = 0; t < 2; ++t) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fw[set][i][t], fa[set][i], acc[t], 0, 0, 0);
+  };
+  fetch(0, s0);
+  for (int s = s0; s < s1; s += 2 * STREAM_STEPS) {
+    fetch(1, s + STREAM_STEPS);
+    multiply(0);
+    if (s + 2 * STREAM_STEPS < s1) fetch(0, s + 2 * STREAM_STEPS);
+    multiply(1);
+  }
+  part[wave][0][lane] = acc[0];
+  part[wave][1][lane] = acc[1];
+  __syncthreads();
+  if (wave >= (FORM == 0 ? 1 : 2) || lr >= count) return;
+  gt_f32x4 sum[2];
+#pragma unroll
+  for (int t = 0; t < 2; ++t) {
+    const int which = FORM == 0 ? t : wave;
+    sum[t] = part[0][which][lane];
+#pragma unroll
+    for (int w = 1; w < 4; ++w) sum[t] += part[w][which][lane];
+    if constexpr (FORM != 0) break;
+  }
+  const int col = n0 + (FORM == 0 ? 0 : wave * 16) + lg * 4;
+  if (col >= N) return;                   // N is a multiple of 8: all four or none
+  if constexpr (FORM == 2) {
+    *(gt_f32x4*)(pair_out + (long long)order[first + lr] * N + col) = sum[0];
+  } else {
+    const float w = in_weights ? in_weights[order[first + lr]] : 1.f;
+    typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
+    bf16x4 out;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      out[i] = (__bf16)(FORM == 0 ? expert_act(w * sum[0][i], w * sum[1][i], limit, alpha) : plain_act(w * sum[0][i], plain));
+    *(bf16x4*)(act + (long long)(first + lr) * N + col) = out;
+  }
+}
+
 // residual[t, :] (+)= sum_j weights[t, j] * pair_out[t * top + j, :], j ascending (weights null: every weight is 1), and
 // what joins a token's experts:
 struct Combine {
@@ -465,22 +567,18 @@ static int launch_combine(const float* pair_out, const float* weights, int num_t
 
 // ---------------------------------------------------------------------------------------------
 extern "C" int vk_moe_max_tiles(int pairs, int experts, int tile_rows) {
-  return (pairs + tile_rows - 1) / tile_rows + experts;
+  return (pairs + tile_rows - 1) / tile_rows + (experts < pairs ? experts : pairs);
 }
 
-// Whether the products of these operands run on the matrix cores (tiles of 128 places) or as 32-bit FMAs (64).
+// Whether the products of these operands run on the matrix cores (tiles of 128 or 16 places) or as 32-bit FMAs (64).
 static inline bool moe_on_matrix_cores(int dtype, int width, int ff, long long ldh) {
   return dtype == DT_BF16 && width % 8 == 0 && ff % 8 == 0 && ldh % 8 == 0;
-}
-
-extern "C" int vk_moe_tile_rows(int dtype, int width, int ff, long long ldh) {
-  return moe_on_matrix_cores(dtype, width, ff, ldh) ? GT_TILE : MOE_TILE;
 }
 
 extern "C" int vk_moe_route(const float* logits, int experts, int top, int num_tokens, int tile_rows, int groups, int keep,
                             int all_scores, const float* correction, float weight_scale, long long ld, int* ids,
                             float* weights, int* offsets, int* order, int* tiles, int* num_tiles, void* stream) {
-  if (tile_rows != MOE_TILE && tile_rows != GT_TILE) return VK_BAD_ARGUMENT;
+  if (tile_rows != MOE_TILE && tile_rows != GT_TILE && tile_rows != MOE_FEW) return VK_BAD_ARGUMENT;
   if (groups < 1 || keep < 1 || keep > groups || experts % groups != 0) return VK_BAD_ARGUMENT;
   if (groups > WAVE) return VK_UNSUPPORTED_SIZE;
   if (keep < groups && (long long)keep * (experts / groups) < top) return VK_BAD_ARGUMENT;
@@ -508,11 +606,11 @@ extern "C" int vk_moe_route(const float* logits, int experts, int top, int num_t
 // accumulate 0: the weighted sums are written to `residual` instead of added to it.  weigh_input: a pair's weight
 // multiplies what its expert reads (w h, applied to the gate and up sums, which are linear in h) instead of what it
 // returns.  plain: 0 experts with a gate (limit, alpha), else experts without one and their activation (plain_act; wg is
-// not read).  extra, extra_gate, stream: see Combine.
+// not read).  extra, extra_gate, stream: see Combine.  tile_rows: what the grouping was made for.
 extern "C" int vk_moe_experts(const void* h, long long ldh, const void* wg, const void* wu, const void* wd, int dtype,
                               const int* offsets, const int* order, const int* tiles, const int* num_tiles,
-                              const float* weights, int num_tokens, int experts, int top, int width, int ff, float limit,
-                              float alpha, int plain, void* act, float* pair_out, float* residual, int accumulate,
+                              const float* weights, int num_tokens, int experts, int top, int width, int ff, int tile_rows,
+                              float limit, float alpha, int plain, void* act, float* pair_out, float* residual, int accumulate,
                               int weigh_input, const float* extra, const float* extra_gate, long long ldg, void* stream_rows,
                               void* stream) {
   if (num_tokens <= 0) return 0;
@@ -524,7 +622,28 @@ extern "C" int vk_moe_experts(const void* h, long long ldh, const void* wg, cons
   hipStream_t s = (hipStream_t)stream;
   const Combine with{extra, extra_gate, ldg, (bf16_t*)stream_rows};
   if (moe_on_matrix_cores(dtype, width, ff, ldh)) {
-    if (((uintptr_t)h | (uintptr_t)wg | (uintptr_t)wu | (uintptr_t)wd | (uintptr_t)act) & 15) return VK_BAD_ARGUMENT;
+    if (((uintptr_t)h | (uintptr_t)wg | (uintptr_t)wu | (uintptr_t)wd | (uintptr_t)act | (uintptr_t)pair_out) & 15)
+      return VK_BAD_ARGUMENT;
+    if (tile_rows == MOE_FEW) {
+      const int few_tiles = vk_moe_max_tiles(pairs, experts, MOE_FEW);
+      if (few_tiles > 65535) return VK_UNSUPPORTED_SIZE;
+      const __bf16 *x = (const __bf16*)h, *g = (const __bf16*)wg, *u = (const __bf16*)wu;
+      if (plain)
+        moe_stream_kernel<1><<<dim3((ff + 31) / 32, few_tiles), 256, 0, s>>>(x, ldh, nullptr, u, offsets, order, tiles, num_tiles,
+                                                                            top, width, ff, limit, alpha, plain, in_weights,
+                                                                            (__bf16*)act, nullptr);
+      else
+        moe_stream_kernel<0><<<dim3((ff + 15) / 16, few_tiles), 256, 0, s>>>(x, ldh, g, u, offsets, order, tiles, num_tiles, top,
+                                                                            width, ff, limit, alpha, 0, in_weights,
+                                                                            (__bf16*)act, nullptr);
+      VK_LAUNCH_CHECK();
+      moe_stream_kernel<2><<<dim3((width + 31) / 32, few_tiles), 256, 0, s>>>((const __bf16*)act, ff, nullptr, (const __bf16*)wd,
+                                                                              offsets, order, tiles, num_tiles, top, ff, width,
+                                                                              limit, alpha, 0, nullptr, nullptr, pair_out);
+      VK_LAUNCH_CHECK();
+      return launch_combine(pair_out, out_weights, num_tokens, top, width, residual, accumulate, with, s);
+    }
+    if (tile_rows != GT_TILE) return VK_BAD_ARGUMENT;
     const int wide_tiles = vk_moe_max_tiles(pairs, experts, GT_TILE), columns = plain ? GT_TILE : 64;
     dim3 up(wide_tiles, (ff + columns - 1) / columns), down(wide_tiles, (width + GT_TILE - 1) / GT_TILE);
     if (up.y > 65535 || down.y > 65535) return VK_UNSUPPORTED_SIZE;
@@ -549,6 +668,7 @@ extern "C" int vk_moe_experts(const void* h, long long ldh, const void* wg, cons
     VK_LAUNCH_CHECK();
     return launch_combine(pair_out, out_weights, num_tokens, top, width, residual, accumulate, with, s);
   }
+  if (tile_rows != MOE_TILE) return VK_BAD_ARGUMENT;
   const int max_tiles = vk_moe_max_tiles(pairs, experts, MOE_TILE);
   dim3 up_grid(max_tiles, (ff + MOE_TILE - 1) / MOE_TILE), down_grid(max_tiles, (width + MOE_TILE - 1) / MOE_TILE);
   if (up_grid.y > 65535 || down_grid.y > 65535) return VK_UNSUPPORTED_SIZE;

@@ -17,17 +17,19 @@ from . import kernels
 
 @dataclass
 class AttentionExtras:
-    """What a layer's softmax and mask have beyond scale, window and cap: ``sink`` ([heads] 32-bit: a learned logit per
+    """What a layer's softmax, mask and output have beyond scale, window and cap: ``sink`` ([heads] 32-bit: a learned logit per
     head that joins the denominator and nothing else), ``rel`` ([heads, far + 1] 32-bit: a bias added to the scaled
-    score by the distance between query and key, the last column for every distance from ``far`` on) and
-    ``keep_first`` (with a window: positions below it stay visible).  The attention kernels take them as they take a
+    score by the distance between query and key, the last column for every distance from ``far`` on),
+    ``keep_first`` (with a window: positions below it stay visible) and ``gate`` ([tokens, >= heads] 32-bit: a head's output
+    is multiplied by the sigmoid of its number; set anew for every step).  The attention kernels take them as they take a
     window."""
     sink: Optional[torch.Tensor] = None
     rel: Optional[torch.Tensor] = None
     keep_first: int = 0
+    gate: Optional[torch.Tensor] = None
 
     def any(self) -> bool:
-        return self.sink is not None or self.rel is not None or self.keep_first > 0
+        return self.sink is not None or self.rel is not None or self.keep_first > 0 or self.gate is not None
 
 
 DECODE_WAVES_WANTED = 512    # enough waves to keep the memory system busy (each keeps a step of loads in flight)

@@ -41,6 +41,7 @@ MODULES: Dict[str, tuple] = {
     "state_space": ("hip", ["kernels/state_space.hip"], ["kernels/common.h"]),
     "streams": ("hip", ["kernels/streams.hip"], ["kernels/common.h"]),
     "latent": ("hip", ["kernels/latent.hip"], ["kernels/common.h", "kernels/group_tile.h"]),
+    "token_side": ("hip", ["kernels/token_side.hip"], ["kernels/common.h"]),
     "moe": ("hip", ["kernels/moe.hip"], ["kernels/common.h", "kernels/group_tile.h"]),
     "host": ("host", ["host/cache_manager.cpp", "host/scheduler.cpp", "host/c_api.cpp"],
              ["host/cache_manager.h", "host/scheduler.h"]),

@@ -280,20 +280,21 @@ def attn_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, 
     if head_dim > ATTENTION_MAX_HEAD_DIM:
         raise UnsupportedError(f"attention: head_dim {head_dim} is above the kernels' limit of {ATTENTION_MAX_HEAD_DIM}")
     fn = _fn("attn_generic", "vk_attn_generic_ext",
-             [_p, _ll, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _i, _f, _p, _p, _p, _i, _i, _p])
+             [_p, _ll, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _i, _f, _p, _p, _p, _i, _i, _p, _ll, _p])
     _status(fn(_ptr(q), q.stride(0), _ptr(k_cache), _ptr(v_cache), _ptr(out), _dt(q, "q"), _ptr(positions),
                _ptr(entry_of_token), _ptr(block_table), block_table.shape[1], k_cache.shape[2], num_tokens, heads,
                kv_heads, head_dim, float(scale), int(window), float(softcap), _ptr(skip_single_of),
-               *attn_extras_args(extras, heads, window), _stream()), "attn_generic")
+               *attn_extras_args(extras, heads, window, out.shape[0]), _stream()), "attn_generic")
 
 
-def attn_extras_args(extras, heads: int, window: int):
-    """``(sink, rel, rel_far, keep_first)`` as the attention launchers take them; ``extras`` (or None) has the
+def attn_extras_args(extras, heads: int, window: int, tokens: int):
+    """``(sink, rel, rel_far, keep_first, gate, gate_ld)`` as the attention launchers take them; ``extras`` (or None) has the
     attributes ``sink`` ([heads] 32-bit or None: a learned logit per head that joins the softmax's denominator only),
     ``rel`` ([heads, rel_far + 1] 32-bit or None: a bias by distance, the last column for every distance from
-    ``rel_far`` on) and ``keep_first`` (positions below it stay visible to a windowed layer)."""
+    ``rel_far`` on), ``keep_first`` (positions below it stay visible to a windowed layer) and ``gate`` ([tokens, >= heads]
+    32-bit or None: a head's output is multiplied by the sigmoid of its number)."""
     if extras is None:
-        return _p(0), _p(0), 0, 0
+        return _p(0), _p(0), 0, 0, _p(0), 0
     sink, rel, keep_first = extras.sink, extras.rel, int(extras.keep_first or 0)
     _dev(sink, rel)
     rel_far = 0
@@ -305,7 +306,12 @@ def attn_extras_args(extras, heads: int, window: int):
               and rel.shape[1] >= 1, "attention: the bias by distance is [heads, distances] in 32-bit")
         rel_far = rel.shape[1] - 1
     _need(keep_first >= 0 and (keep_first == 0 or window > 0), "attention: kept first positions need a window")
-    return _ptr(sink), _ptr(rel), rel_far, keep_first
+    gate = extras.gate
+    if gate is not None:
+        _dev(gate)
+        _need(gate.dtype == torch.float32 and gate.dim() == 2 and gate.stride(1) == 1 and gate.shape[0] >= tokens
+              and gate.shape[1] >= heads, "attention: one 32-bit gate per token and query head")
+    return _ptr(sink), _ptr(rel), rel_far, keep_first, _ptr(gate), gate.stride(0) if gate is not None else 0
 
 
 ATTN_DECODE_F32_CHUNK = 256   # positions of one workgroup of attn_decode_f32 (the kernel's DEC_CHUNK)
@@ -341,11 +347,11 @@ def attn_decode_f32(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
           "attention: entry arrays")
     _need(heads % kv_heads == 0 and chunks >= 1, "attention: heads must be a multiple of kv_heads")
     fn = _fn("attn_generic", "vk_attn_decode_f32_ext",
-             [_p, _ll, _p, _p, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _f, _i, _f, _i, _p, _p, _i, _i, _p])
+             [_p, _ll, _p, _p, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _f, _i, _f, _i, _p, _p, _i, _i, _p, _ll, _p])
     _status(fn(_ptr(q), q.stride(0), _ptr(k_cache), _ptr(v_cache), _ptr(out), _ptr(partial), _ptr(entries), count,
                _ptr(entry_start), _ptr(entry_first_pos), _ptr(block_table), block_table.shape[1], k_cache.shape[2],
                heads, kv_heads, head_dim, float(scale), int(window), float(softcap), int(chunks),
-               *attn_extras_args(extras, heads, window), _stream()), "attn_decode_f32")
+               *attn_extras_args(extras, heads, window, out.shape[0]), _stream()), "attn_decode_f32")
 
 
 ATTN_PREFILL_F32_MAX_HEAD_DIM = 128   # the K, V and weight tiles of a wider head do not fit a CU's LDS
@@ -379,11 +385,11 @@ def attn_prefill_f32(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
           "attention: entry arrays")
     _need(heads % kv_heads == 0, "attention: heads must be a multiple of kv_heads")
     fn = _fn("attn_generic", "vk_attn_prefill_f32_ext",
-             [_p, _ll, _p, _p, _p, _p, _i, _i, _p, _p, _p, _i, _i, _i, _i, _i, _f, _i, _f, _p, _p, _i, _i, _p])
+             [_p, _ll, _p, _p, _p, _p, _i, _i, _p, _p, _p, _i, _i, _i, _i, _i, _f, _i, _f, _p, _p, _i, _i, _p, _ll, _p])
     _status(fn(_ptr(q), q.stride(0), _ptr(k_cache), _ptr(v_cache), _ptr(out), _ptr(tiles), tiles.numel() // 2,
                int(tile_tokens), _ptr(entry_start), _ptr(entry_first_pos), _ptr(block_table), block_table.shape[1],
                k_cache.shape[2], heads, kv_heads, head_dim, float(scale), int(window), float(softcap),
-               *attn_extras_args(extras, heads, window), _stream()), "attn_prefill_f32")
+               *attn_extras_args(extras, heads, window, out.shape[0]), _stream()), "attn_prefill_f32")
 
 
 # ----------------------------------------------------------------------------------------------
@@ -782,13 +788,13 @@ def attn_bf16_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
         chunk_tiles = max_chunks = 0
     module = f"attn_bf16_hd{attn_bf16_padded_width(head_dim)}"
     fn = _fn(module, "vk_attn_bf16_prefill_ext",
-             [_p, _ll, _p, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _f, _i, _f, _i, _p, _ll, _i, _i, _p, _p, _i, _i, _p],
+             [_p, _ll, _p, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _f, _i, _f, _i, _p, _ll, _i, _i, _p, _p, _i, _i, _p, _ll, _p],
              key=module + ".prefill")
     _status(fn(_ptr(q), q.stride(0), _ptr(k_cache), _ptr(v_cache), _ptr(out), _ptr(tiles), num_tiles,
                _ptr(entry_start), _ptr(entry_first_pos), _ptr(block_table), block_table.shape[1], k_cache.shape[2],
                heads, kv_heads, head_dim, float(scale), int(window), float(softcap), 1 if split else 0, _ptr(partial),
                partial.numel() if partial is not None else 0, int(chunk_tiles), int(max_chunks),
-               *attn_extras_args(extras, heads, window), _stream()),
+               *attn_extras_args(extras, heads, window, out.shape[0]), _stream()),
             "attn_bf16_prefill")
 
 
@@ -821,12 +827,12 @@ def attn_bf16_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
     _need(block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.is_contiguous(), "attention: table")
     module = f"attn_bf16_hd{attn_bf16_padded_width(head_dim)}"
     fn = _fn(module, "vk_attn_bf16_decode_ext",
-             [_p, _ll, _p, _p, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _f, _i, _f, _i, _i, _i, _i, _p, _p, _i, _i, _p],
+             [_p, _ll, _p, _p, _p, _p, _p, _i, _p, _p, _p, _i, _i, _i, _i, _i, _f, _i, _f, _i, _i, _i, _i, _p, _p, _i, _i, _p, _ll, _p],
              key=module + ".decode")
     _status(fn(_ptr(q), q.stride(0), _ptr(k_cache), _ptr(v_cache), _ptr(out), _ptr(partial), _ptr(entries), count,
                _ptr(entry_start), _ptr(entry_first_pos), _ptr(block_table), block_table.shape[1], k_cache.shape[2],
                heads, kv_heads, head_dim, float(scale), int(window), float(softcap), int(chunk), int(chunks), 1 if dense else 0,
-               1 if join else 0, *attn_extras_args(extras, heads, window), _stream()),
+               1 if join else 0, *attn_extras_args(extras, heads, window, out.shape[0]), _stream()),
             "attn_bf16_decode")
 
 
@@ -1292,14 +1298,20 @@ def head_linear(a: torch.Tensor, a_head_stride: int, k: int, w: torch.Tensor, ou
 
 
 # --- mixture of experts ---------------------------------------------------------------------------
-def moe_tile_rows(h: torch.Tensor, width: int, ff: int) -> int:
-    """Places per tile of the experts' products for activations ``h``: 128 on the matrix cores (bfloat16, widths that
-    are multiples of 8), 64 as 32-bit FMAs.  The grouping has to be made for the same number."""
-    return 128 if (h.dtype == torch.bfloat16 and width % 8 == 0 and ff % 8 == 0 and h.stride(0) % 8 == 0) else 64
+MOE_STREAM_PAIRS = 16     # pairs per expert, on average, up to which the experts' products are streams of the weights
+
+
+def moe_tile_rows(h: torch.Tensor, width: int, ff: int, pairs: int, experts: int) -> int:
+    """Places per tile of the experts' products for activations ``h`` of ``pairs`` (token, choice) pairs: on the matrix cores
+    (bfloat16, widths that are multiples of 8) 128, or 16 where few pairs fall to an expert; 64 as 32-bit FMAs.  The grouping
+    has to be made for the same number."""
+    if not (h.dtype == torch.bfloat16 and width % 8 == 0 and ff % 8 == 0 and h.stride(0) % 8 == 0):
+        return 64
+    return 16 if pairs <= MOE_STREAM_PAIRS * experts else 128
 
 
 def moe_max_tiles(pairs: int, experts: int, tile_rows: int = 64) -> int:
-    return (pairs + tile_rows - 1) // tile_rows + experts
+    return (pairs + tile_rows - 1) // tile_rows + min(pairs, experts)
 
 
 def moe_route(logits: torch.Tensor, top: int, ids: torch.Tensor, weights: torch.Tensor, offsets: torch.Tensor,
@@ -1321,7 +1333,7 @@ def moe_route(logits: torch.Tensor, top: int, ids: torch.Tensor, weights: torch.
     _f32(weights, "moe_route: weights")
     _need(ids.numel() == tokens * top and weights.numel() == tokens * top and order.numel() == tokens * top
           and offsets.numel() == experts + 1 and tiles.numel() >= 2 * moe_max_tiles(tokens * top, experts, tile_rows)
-          and num_tiles.numel() == 1 and tile_rows in (64, 128), "moe_route: output sizes")
+          and num_tiles.numel() == 1 and tile_rows in (16, 64, 128), "moe_route: output sizes")
     _need(1 <= keep <= groups <= 64 and experts % groups == 0 and (keep == groups or keep * (experts // groups) >= top),
           f"moe_route: {keep} of {groups} groups of {experts} experts for top {top}")
     mode = {"sigmoid": 2, "steered": 3}.get(all_scores, 1 if all_scores else 0)
@@ -1338,7 +1350,7 @@ def moe_route(logits: torch.Tensor, top: int, ids: torch.Tensor, weights: torch.
 def moe_experts(h: torch.Tensor, w_gate: Optional[torch.Tensor], w_up: torch.Tensor, w_down: torch.Tensor, offsets: torch.Tensor,
                 order: torch.Tensor, tiles: torch.Tensor, num_tiles: torch.Tensor, weights: torch.Tensor, top: int,
                 limit: float, alpha: float, act: torch.Tensor, pair_out: torch.Tensor, residual: torch.Tensor,
-                accumulate: bool = True, weigh_input: bool = False, plain: Optional[str] = None,
+                accumulate: bool = True, weigh_input: bool = False, tile_rows: int = 128, plain: Optional[str] = None,
                 extra: Optional[torch.Tensor] = None, extra_gate: Optional[torch.Tensor] = None,
                 stream: Optional[torch.Tensor] = None) -> None:
     """The chosen experts of every token: ``y = g * sigmoid(alpha * g) * (u + 1)`` with ``g = min(Wg h, limit)`` and
@@ -1374,13 +1386,14 @@ def moe_experts(h: torch.Tensor, w_gate: Optional[torch.Tensor], w_up: torch.Ten
           "moe_experts: output shapes")
     _i32(offsets, order, tiles, num_tiles)
     _need(offsets.numel() == experts + 1 and order.numel() == tokens * top
-          and tiles.numel() >= 2 * moe_max_tiles(tokens * top, experts, moe_tile_rows(h, width, ff)),
-          "moe_experts: grouping (made by moe_route with moe_tile_rows(h, width, ff))")
-    fn = _fn("moe", "vk_moe_experts", [_p, _ll, _p, _p, _p, _i, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _f, _f, _i, _p, _p,
+          and tiles.numel() >= 2 * moe_max_tiles(tokens * top, experts, tile_rows)
+          and (tile_rows == 64) == (moe_tile_rows(h, width, ff, 0, 1) == 64) and tile_rows in (16, 64, 128),
+          "moe_experts: grouping (made by moe_route with the tile_rows that moe_tile_rows gives)")
+    fn = _fn("moe", "vk_moe_experts", [_p, _ll, _p, _p, _p, _i, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _f, _i, _p, _p,
                                        _p, _i, _i, _p, _p, _ll, _p, _p])
     _status(fn(_ptr(h), h.stride(0), _ptr(w_gate), _ptr(w_up), _ptr(w_down), _dt(h, "h"), _ptr(offsets), _ptr(order),
-               _ptr(tiles), _ptr(num_tiles), _ptr(weights), tokens, experts, top, width, ff, float(limit), float(alpha),
-               ACTIVATIONS[plain] if plain else 0, _ptr(act), _ptr(pair_out), _ptr(residual), 1 if accumulate else 0,
+               _ptr(tiles), _ptr(num_tiles), _ptr(weights), tokens, experts, top, width, ff, int(tile_rows),
+               float(limit), float(alpha), ACTIVATIONS[plain] if plain else 0, _ptr(act), _ptr(pair_out), _ptr(residual), 1 if accumulate else 0,
                1 if weigh_input else 0, _ptr(extra), _ptr(extra_gate), extra_gate.stride(0) if extra_gate is not None else 0,
                _ptr(stream), _stream()),
             "moe_experts")
@@ -1418,6 +1431,44 @@ def rmsnorm_add(y: torch.Tensor, weight: torch.Tensor, eps: float, residual: tor
     fn = _fn("elementwise", "vk_rmsnorm_add", [_p, _p, _p, _i, _i, _f, _p, _p, _f, _i, _p, _i, _p])
     _status(fn(_ptr(y), _ptr(weight), _ptr(residual), rows, width, float(eps), _ptr(next_weight), _ptr(next_bias),
                float(next_eps), 1 if next_kind == "layer" else 0, _ptr(next_out), _dt(next_out, "next_out") if next_out is not None else 0, _stream()), "rmsnorm_add")
+
+
+TOKEN_SIDE_MAX_TOKENS = 256          # a workgroup per token: one for every CU
+TOKEN_SIDE_MAX_BYTES = 144 * 1024    # LDS of a workgroup: six bytes a column of the stream, four a number of the gate
+
+
+def token_side_supported(x: torch.Tensor, gate: torch.Tensor, proj: torch.Tensor) -> bool:
+    """Whether :func:`token_side` takes the operands: bfloat16 weights, widths that are multiples of 8 and fit the LDS,
+    and so few tokens that a workgroup per token does not read the weights too often."""
+    dim, width = gate.shape
+    return (x.shape[0] <= TOKEN_SIDE_MAX_TOKENS and gate.dtype == torch.bfloat16 and proj.dtype == torch.bfloat16
+            and width % 8 == 0 and dim % 8 == 0 and 6 * width + 4 * dim <= TOKEN_SIDE_MAX_BYTES)
+
+
+def token_side(x: torch.Tensor, e: torch.Tensor, gate: torch.Tensor, proj: torch.Tensor, norm: torch.Tensor, eps: float,
+               next_out: Optional[torch.Tensor] = None, next_weight: Optional[torch.Tensor] = None, next_eps: float = 0.0,
+               next_kind: str = "rms", next_bias: Optional[torch.Tensor] = None) -> None:
+    """``y = proj (gelu_tanh(gate x) * e); x += y / sqrt(mean(y^2) + eps) * norm`` for every row of the 32-bit stream ``x``
+    (``e [tokens, dim]``: 32-bit, may be a view of some columns), and the next norm of the new rows into ``next_out`` as
+    :func:`rmsnorm_add` applies it.  One launch, a workgroup per token."""
+    _dev(x, e, gate, proj, norm, next_out, next_weight, next_bias)
+    _need(token_side_supported(x, gate, proj), "token_side: operands")
+    tokens, width = x.shape
+    dim = gate.shape[0]
+    _f32(x, "token_side: x")
+    _f32s(e, "token_side: e")
+    _need(x.is_contiguous() and e.shape == (tokens, dim) and gate.is_contiguous() and proj.shape == (width, dim)
+          and proj.is_contiguous(), "token_side: shapes")
+    for t, what in ((norm, "norm"), (next_weight, "next_weight"), (next_bias, "next_bias")):
+        if t is not None:
+            _need(t.dtype == torch.float32 and t.numel() == width and t.is_contiguous(), f"token_side: {what}")
+    if next_out is not None:
+        _need(next_weight is not None and next_kind in ("rms", "layer") and next_out.shape == x.shape
+              and next_out.is_contiguous() and next_out.dtype == torch.bfloat16, "token_side: next_out")
+    fn = _fn("token_side", "vk_token_side", [_p, _p, _ll, _p, _p, _p, _f, _p, _p, _f, _i, _p, _i, _i, _i, _p])
+    _status(fn(_ptr(x), _ptr(e), e.stride(0), _ptr(gate), _ptr(proj), _ptr(norm), float(eps), _ptr(next_weight),
+               _ptr(next_bias), float(next_eps), 1 if next_kind == "layer" else 0, _ptr(next_out), tokens, width, dim,
+               _stream()), "token_side")
 
 
 def axpby(x: torch.Tensor, a: float, y: torch.Tensor, b: float, out: torch.Tensor, accumulate: bool = False) -> None:

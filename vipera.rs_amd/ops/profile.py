@@ -28,7 +28,7 @@ LAUNCHERS = (
     "attn_bf16_decode", "gemm_bf16_mid", "gemm_bf16_gated", "gemm_bf16_gated_act", "gemm_bf16_gated_tile_scaled",
     "dyt", "scale_", "tanh", "decay_", "delta_prepare", "delta_rule", "wkv_rule", "token_shift", "head_norm_gate",
     "latent_prepare", "latent_q_rotate", "head_linear", "moe_route", "moe_experts",
-    "rmsnorm_add", "axpby", "activation", "whole_norm_pack", "head_unpack_gate", "decay_rule", "gated_norm",
+    "rmsnorm_add", "token_side", "axpby", "activation", "whole_norm_pack", "head_unpack_gate", "decay_rule", "gated_norm",
     "causal_conv", "selective_scan", "scan_prepare", "head_norm_pack", "channel_decay", "memory_rule", "dyt_pair",
     "head_prepare", "head_conv_prepare", "head_finish", "rotate_scale", "row_gate_add", "streams_step", "state_space", "gated_part_norm",
 )

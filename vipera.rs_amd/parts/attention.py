@@ -378,19 +378,25 @@ class Attention(Mixer):
             kernels.rope_kvwrite(qkv, batch.positions, inv_freq, rotary_dim, None, None, batch.entry_of_token, None,
                                  heads, self.kv_heads, width, angles)
         attn = self.runtime.empty((tokens, heads * width))
+        gate = proj[:, self.gate_col:] if self.gate else None
+        # one gate per head rides in the attention kernels; two maps' difference is gated behind it
+        rides = self.gate == "head_sigmoid" and self.maps == 1
+        if rides:
+            self.extras.gate = gate
         paged_attention(qkv, cache.k, cache.v, attn, batch, table, heads, self.kv_heads, width, self.scale,
                         self.mask, self.softcap, self.extras)
-        if self.maps == 1 and not self.gate and width == self.value_dim:      # nothing to unpack
+        self.extras.gate = None
+        if self.maps == 1 and (rides or not self.gate) and width == self.value_dim:      # nothing to unpack
             linear(attn, self.w_o, self.b_o, residual, accumulate=accumulate)
             return
         values = self.runtime.empty((tokens, self.heads * self.value_dim))
-        gate = proj[:, self.gate_col:] if self.gate else None
-        if self.maps > 1 or self.gate == "head_sigmoid":
+        if self.maps > 1:
             kernels.head_finish(attn, values, self.heads, self.value_dim, width, self.maps, self.subtract,
-                                unit_norm=self.maps > 1, eps=eps, factor=1.0 - self.diff if self.maps > 1 else 1.0,
+                                unit_norm=True, eps=eps, factor=1.0 - self.diff,
                                 gate=gate, gate_kind="sigmoid" if self.gate else "none", gate_per_head=True)
         else:
-            kernels.head_unpack_gate(attn, gate, self.gate or "none", self.heads, self.value_dim, width, values)
+            kernels.head_unpack_gate(attn, None if rides else gate, "none" if rides else self.gate or "none", self.heads,
+                                     self.value_dim, width, values)
         linear(values, self.w_o, self.b_o, residual, accumulate=accumulate)
 
     def forward(self, h, batch, cache, state, position, residual, reads_only: bool = False, handoff=None,

@@ -199,6 +199,11 @@ class FeedForward(Part):
     #: and leaves the new rows of the residual in it
     leaves_stream = False
 
+    def wants_stream(self, residual) -> bool:
+        """Whether ``forward``'s ``h`` may be the stream itself in the run's dtype, and saves work if it is (a part that
+        stands behind both sublayers, see the blocks' ``after``)."""
+        return False
+
     #: a part that sets this takes ``following=`` (a :class:`FollowingNorm`) in ``forward`` and may fill it
     applies_following = False
 

@@ -100,8 +100,7 @@ class PreNormBlock(Block):
         stream = None
         if self.ffn is not None:
             ffn_kwargs = {"outgoing": outgoing} if self.after is None and outgoing is not None and self.ffn.fills_handoff else {}
-            if self.after is not None and self.ffn.leaves_stream and getattr(self.after, "reads_stream_input", False) \
-                    and self.runtime.dtype != torch.float32:
+            if self.after is not None and self.ffn.leaves_stream and self.after.wants_stream(x):
                 stream = ffn_kwargs["stream"] = self.runtime.empty(tuple(x.shape))
             if between is not None and between.groups:
                 self.ffn.forward(None, batch, x, handoff=between, **ffn_kwargs)
@@ -242,7 +241,7 @@ class SandwichBlock(Block):
             y = torch.zeros_like(x)
             parts["mixer"].forward(h, batch, cache, state, parts["position"], y, reads_only)
         after = parts.get("after")
-        feeds_after = after is not None and getattr(after, "reads_stream_input", False)
+        feeds_after = after is not None and after.wants_stream(x)
         if not self.has_ffn:
             stream = parts["mixer_post_norm"].add_into(y, x, as_input=feeds_after)
         else:

@@ -102,10 +102,9 @@ class TokenSide(FeedForward):
     """What a layer adds to the stream from its own columns of the per-token side table (see :class:`Embedding`):
     ``e = side[token][index * dim : (index + 1) * dim]``, ``g = gelu_tanh(Wgate x) * e``, ``y = Wproj g``,
     ``x += y / rms(y) * norm``.  It reads the stream ``x`` itself: ``h`` is the stream in the run's dtype if the block
-    has it at hand (``reads_stream_input``), else it is made here.  ``params``: ``hidden``,
+    has it at hand (``wants_stream``), else it is made here.  ``params``: ``hidden``,
     ``dim``, ``index``, ``eps``, ``activation`` ("gelu_tanh" unless given), ``name``; tensors ``<name>.gate | proj | norm``."""
 
-    reads_stream_input = True     # forward's ``h`` may be the residual itself in the run's dtype
     applies_following = True
 
     def __init__(self, spec: PartSpec, prefix: str, runtime):
@@ -127,11 +126,31 @@ class TokenSide(FeedForward):
         base = f"{self.prefix}{self.spec.params['name']}."
         self.w_gate, self.w_proj, self.norm = tensors[base + "gate"], tensors[base + "proj"], tensors[base + "norm"]
 
+    def takes_few(self, residual) -> bool:
+        """Whether the step runs as one launch that reads the 32-bit stream itself."""
+        return (self.runtime.dtype == torch.bfloat16 and self.activation == "gelu_tanh"
+                and kernels.token_side_supported(residual, self.w_gate, self.w_proj))
+
+    def wants_stream(self, residual) -> bool:
+        """Whether ``forward`` reads ``h``, the stream in the run's dtype."""
+        return self.runtime.dtype != torch.float32 and not self.takes_few(residual)
+
     def forward(self, h, batch, residual, following=None, **_unused) -> None:
         tokens = residual.shape[0]
         rows = batch.shared.get(SIDE_ROWS)
         if rows is None or rows.shape[1] < (self.index + 1) * self.dim:
             raise InvalidArgumentError("token_side: the embedding has left no side rows for this layer in the step")
+        e = rows[:, self.index * self.dim:(self.index + 1) * self.dim]
+        # the norm that follows, if the part behind asks for it and its kind is one the kernels apply
+        fused = following.norm.as_kernel() if following is not None else None
+        after = {}
+        if fused is not None:
+            kind, weight, bias, eps = fused
+            following.out = self.runtime.empty((tokens, self.hidden))
+            after = dict(next_out=following.out, next_weight=weight, next_eps=eps, next_kind=kind, next_bias=bias)
+        if self.takes_few(residual):
+            kernels.token_side(residual, e, self.w_gate, self.w_proj, self.norm, self.eps, **after)
+            return
         x = h if h is not None else residual
         if h is None and self.runtime.dtype != torch.float32:
             x = self.runtime.empty((tokens, self.hidden))
@@ -139,16 +158,10 @@ class TokenSide(FeedForward):
         gate = torch.empty((tokens, self.dim), dtype=torch.float32, device=residual.device)
         linear(x, self.w_gate, None, gate)
         gated = self.runtime.empty((tokens, self.dim))
-        kernels.activation(gate, self.activation, gated, mul=rows[:, self.index * self.dim:(self.index + 1) * self.dim])
+        kernels.activation(gate, self.activation, gated, mul=e)
         y = torch.empty((tokens, self.hidden), dtype=torch.float32, device=residual.device)
         linear(gated, self.w_proj, None, y)
-        fused = following.norm.as_kernel() if following is not None else None
-        if fused is None or fused[0] == "none":
-            kernels.rmsnorm_add(y, self.norm, self.eps, residual)
-            return
-        kind, weight, bias, eps = fused
-        following.out = self.runtime.empty((tokens, self.hidden))
-        kernels.rmsnorm_add(y, self.norm, self.eps, residual, following.out, weight, eps, next_kind=kind, next_bias=bias)
+        kernels.rmsnorm_add(y, self.norm, self.eps, residual, **after)
 
 
 class LMHead(Part):

@@ -150,10 +150,13 @@ class PlainMLP(FeedForward):
         self.w_up, self.w_down = tensors[up], tensors[down]
 
     def forward(self, h, batch, residual, accumulate: bool = True, **_unused) -> None:
-        tokens = residual.shape[0]
-        up = self.runtime.empty((tokens, self.inter))
+        up = self.runtime.empty((residual.shape[0], self.inter))
         linear(h, self.w_up, None, up)
-        act = self.runtime.empty((tokens, self.inter))
+        self.finish(up, residual, accumulate)
+
+    def finish(self, up, residual, accumulate: bool = True) -> None:
+        """The rest, from the up product's sums on (``up`` may be a view of some columns of a larger product)."""
+        act = self.runtime.empty((residual.shape[0], self.inter))
         kernels.activation(up, self.activation, act)
         linear(act, self.w_down, None, residual, accumulate=accumulate)
 

@@ -31,6 +31,7 @@ from ..errors import InvalidArgumentError, UnsupportedError
 from ..ops import kernels
 from ..ops.linear import linear
 from ..weights.checkpoint import MATRIX, VECTOR, TensorSpec
+from .attention import _cat
 from .base import FeedForward, part_class, register_ffn
 
 
@@ -53,6 +54,7 @@ class MixtureOfExperts(FeedForward):
         self.weight_scale = float(p.get("weight_scale", 1.0))
         self.shared_gate = p.get("shared_gate")
         self.correction = self.w_shared_gate = self.b_router = None
+        self.router_col = 0       # where the router's logits begin in the one product
         self.plain = p.get("activation", "relu2") if p.get("form") == "plain" else None
         self.weigh_input = p.get("weigh", "output") == "input"
         self.shared = None
@@ -134,10 +136,14 @@ class MixtureOfExperts(FeedForward):
             if self.shared_gate:
                 # the gate's row rides behind the router's rows: one product for all that is one number per token
                 self.w_shared_gate = tensors[base + "shared.sg"]
-                self.w_router = torch.cat([self.w_router.to(self.w_shared_gate.dtype), self.w_shared_gate]).contiguous()
+                self.w_router = _cat([self.w_router, self.w_shared_gate])
+            if self.plain is not None and self.shared_gate:
+                # and the shared expert's up rows in front of them, which read the same rows
+                self.w_router = _cat([self.shared.w_up, self.w_router])
+                self.router_col, self.shared.w_up = self.shared.inter, None
         if self.spec.params.get("router_bias"):
             bias = torch.zeros(self.w_router.shape[0], dtype=torch.float32, device=self.w_router.device)
-            bias[:self.experts] = tensors[base + self.spec.params["router_bias"]].float()
+            bias[self.router_col:self.router_col + self.experts] = tensors[base + self.spec.params["router_bias"]].float()
             self.b_router = bias
 
     can_overwrite = True
@@ -149,8 +155,8 @@ class MixtureOfExperts(FeedForward):
         pairs = tokens * self.top
         rows = torch.empty((tokens, self.w_router.shape[0]), dtype=torch.float32, device=device)
         linear(h, self.w_router, self.b_router, rows)
-        logits = rows[:, :self.experts]
-        tile_rows = kernels.moe_tile_rows(h, self.hidden, self.inter)
+        logits = rows[:, self.router_col:self.router_col + self.experts]
+        tile_rows = kernels.moe_tile_rows(h, self.hidden, self.inter, pairs, self.experts)
         ints = torch.empty(2 * pairs + self.experts + 2 + 2 * kernels.moe_max_tiles(pairs, self.experts, tile_rows),
                            dtype=torch.int32, device=device)
         ids, order = ints[:pairs], ints[pairs:2 * pairs]
@@ -167,14 +173,17 @@ class MixtureOfExperts(FeedForward):
         if self.shared is not None and self.w_shared_gate is not None:
             # the shared expert into a buffer of its own, which joins the others' sum times the token's gate
             extra = torch.empty_like(residual)
-            self.shared.forward(h, batch, extra, accumulate=False)
+            if self.router_col:
+                self.shared.finish(rows[:, :self.router_col], extra, accumulate=False)
+            else:
+                self.shared.forward(h, batch, extra, accumulate=False)
         elif self.shared is not None:
             # its output lies in the residual already when the experts' sum joins
             self.shared.forward(h, batch, residual, accumulate=accumulate)
             accumulate = True
         kernels.moe_experts(h, self.w_gate, self.w_up, self.w_down, offsets, order, tiles, num_tiles, weights,
                             self.top, self.limit, self.alpha, act, pair_out, residual, accumulate, self.weigh_input,
-                            plain=self.plain, extra=extra, extra_gate=rows[:, self.experts:] if extra is not None else None,
+                            tile_rows, plain=self.plain, extra=extra, extra_gate=rows[:, self.router_col + self.experts:] if extra is not None else None,
                             stream=stream)
 
 
