@@ -1298,7 +1298,7 @@ def head_linear(a: torch.Tensor, a_head_stride: int, k: int, w: torch.Tensor, ou
 
 
 # --- mixture of experts ---------------------------------------------------------------------------
-MOE_STREAM_PAIRS = 16     # pairs per expert, on average, up to which the experts' products are streams of the weights
+MOE_STREAM_PAIRS = 10     # pairs per expert, on average, up to which the experts' products are streams of the weights
 
 
 def moe_tile_rows(h: torch.Tensor, width: int, ff: int, pairs: int, experts: int) -> int:
@@ -1434,7 +1434,7 @@ def rmsnorm_add(y: torch.Tensor, weight: torch.Tensor, eps: float, residual: tor
 
 
 TOKEN_SIDE_MAX_TOKENS = 256          # a workgroup per token: one for every CU
-TOKEN_SIDE_MAX_BYTES = 144 * 1024    # LDS of a workgroup: six bytes a column of the stream, four a number of the gate
+TOKEN_SIDE_MAX_WIDTH = 8_192         # a row stays in a workgroup's registers
 
 
 def token_side_supported(x: torch.Tensor, gate: torch.Tensor, proj: torch.Tensor) -> bool:
@@ -1442,7 +1442,7 @@ def token_side_supported(x: torch.Tensor, gate: torch.Tensor, proj: torch.Tensor
     and so few tokens that a workgroup per token does not read the weights too often."""
     dim, width = gate.shape
     return (x.shape[0] <= TOKEN_SIDE_MAX_TOKENS and gate.dtype == torch.bfloat16 and proj.dtype == torch.bfloat16
-            and width % 8 == 0 and dim % 8 == 0 and 6 * width + 4 * dim <= TOKEN_SIDE_MAX_BYTES)
+            and width % 8 == 0 and dim % 8 == 0 and width <= TOKEN_SIDE_MAX_WIDTH)
 
 
 def token_side(x: torch.Tensor, e: torch.Tensor, gate: torch.Tensor, proj: torch.Tensor, norm: torch.Tensor, eps: float,
@@ -1450,7 +1450,7 @@ def token_side(x: torch.Tensor, e: torch.Tensor, gate: torch.Tensor, proj: torch
                next_kind: str = "rms", next_bias: Optional[torch.Tensor] = None) -> None:
     """``y = proj (gelu_tanh(gate x) * e); x += y / sqrt(mean(y^2) + eps) * norm`` for every row of the 32-bit stream ``x``
     (``e [tokens, dim]``: 32-bit, may be a view of some columns), and the next norm of the new rows into ``next_out`` as
-    :func:`rmsnorm_add` applies it.  One launch, a workgroup per token."""
+    :func:`rmsnorm_add` applies it.  Two launches: the gated numbers, then the rest with a workgroup per token."""
     _dev(x, e, gate, proj, norm, next_out, next_weight, next_bias)
     _need(token_side_supported(x, gate, proj), "token_side: operands")
     tokens, width = x.shape
@@ -1465,10 +1465,11 @@ def token_side(x: torch.Tensor, e: torch.Tensor, gate: torch.Tensor, proj: torch
     if next_out is not None:
         _need(next_weight is not None and next_kind in ("rms", "layer") and next_out.shape == x.shape
               and next_out.is_contiguous() and next_out.dtype == torch.bfloat16, "token_side: next_out")
-    fn = _fn("token_side", "vk_token_side", [_p, _p, _ll, _p, _p, _p, _f, _p, _p, _f, _i, _p, _i, _i, _i, _p])
+    fn = _fn("token_side", "vk_token_side", [_p, _p, _ll, _p, _p, _p, _f, _p, _p, _f, _i, _p, _p, _i, _i, _i, _p])
+    g = torch.empty((tokens, dim), dtype=torch.bfloat16, device=x.device)
     _status(fn(_ptr(x), _ptr(e), e.stride(0), _ptr(gate), _ptr(proj), _ptr(norm), float(eps), _ptr(next_weight),
-               _ptr(next_bias), float(next_eps), 1 if next_kind == "layer" else 0, _ptr(next_out), tokens, width, dim,
-               _stream()), "token_side")
+               _ptr(next_bias), float(next_eps), 1 if next_kind == "layer" else 0, _ptr(next_out), _ptr(g),
+               tokens, width, dim, _stream()), "token_side")
 
 
 def axpby(x: torch.Tensor, a: float, y: torch.Tensor, b: float, out: torch.Tensor, accumulate: bool = False) -> None:

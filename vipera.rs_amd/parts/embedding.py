@@ -127,7 +127,7 @@ class TokenSide(FeedForward):
         self.w_gate, self.w_proj, self.norm = tensors[base + "gate"], tensors[base + "proj"], tensors[base + "norm"]
 
     def takes_few(self, residual) -> bool:
-        """Whether the step runs as one launch that reads the 32-bit stream itself."""
+        """Whether the step runs on the kernels for few tokens, which read the 32-bit stream itself."""
         return (self.runtime.dtype == torch.bfloat16 and self.activation == "gelu_tanh"
                 and kernels.token_side_supported(residual, self.w_gate, self.w_proj))
 
