@@ -239,6 +239,21 @@ def test_every_pass_reads_the_layers_own_columns_of_the_side_table():
     assert [bool(np.allclose(a, b)) for a, b in zip(got, want)] == [True, True, False, False, False, False]
 
 
+def test_a_plan_counts_a_looped_layers_weights_once_a_pass(tmp_path):
+    from vipera_rs_amd.cli import plan_model
+    from vipera_rs_amd.models import tensor_reads
+
+    reads = tensor_reads(config_from_dict(Z.R1))
+    assert (reads["l0.mix.q"], reads["l1.mix.q"], reads["l2.mlp.e3.up"], reads["l3.mix.o"], reads["loop.in"]) == (1, 2, 2, 1, 2)
+    steps = [plan_model(Z.make_folder(tmp_path / str(times), dict(Z.R1, loop={"start": 1, "stop": 3, "times": times}), 3), 64, 1,
+                        "bfloat16", 16)["decode_step_read_bytes"] for times in (1, 2, 3)]
+    kept = [n for n in declare_cache_needs(config_from_dict(Z.R1))[1:3]]
+    per_pass = sum(2 * math.prod(s.shape) for s in declare_model(config_from_dict(Z.R1))
+                   if s.role == "matrix" and (s.name.startswith(("l1.", "l2.")) or s.name == "loop.in"))
+    per_pass += sum(64 * n.kv.bytes_per_position(2) + n.state.bytes_per_slot() for n in kept)
+    assert steps[1] - steps[0] == steps[2] - steps[1] == per_pass
+
+
 def test_model_info_names_the_architecture(tmp_path):
     folder = Z.make_folder(tmp_path / "r2", Z.R2, 5)
     root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))

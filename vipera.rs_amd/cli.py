@@ -193,7 +193,7 @@ def plan_model(folder: str, ctx: Optional[int], batch: int, dtype: str, block_si
 
     from .cache import cache_bytes
     from .config.registry import load_config
-    from .models import check_model, declare_cache_needs, declare_model
+    from .models import check_model, declare_cache_needs, declare_model, tensor_reads
     from .weights.checkpoint import MATRIX, Checkpoint, kept_bytes, kept_dtype
 
     config = load_config(folder)
@@ -212,6 +212,7 @@ def plan_model(folder: str, ctx: Optional[int], batch: int, dtype: str, block_si
     try:
         weight_bytes = kept_bytes(checkpoint, specs, run_dtype, keep_float32)
         matrix_elements = matrix_bytes = 0
+        reads = tensor_reads(config)
         for spec in specs:
             present = spec.name in checkpoint.tensors
             if spec.role != MATRIX or (spec.optional and not present):
@@ -219,6 +220,7 @@ def plan_model(folder: str, ctx: Optional[int], batch: int, dtype: str, block_si
             count = 1
             for dim in (checkpoint.info(spec.name).shape if present else spec.shape):
                 count *= max(int(dim), 0)
+            count *= reads.get(spec.name, 1)      # a layer that runs several times is read that often
             matrix_elements += count
             stored = checkpoint.info(spec.name).torch_dtype if present else run_dtype
             matrix_bytes += count * (4 if kept_dtype(spec, stored, run_dtype, keep_float32) == torch.float32 else 2)
@@ -235,7 +237,7 @@ def plan_model(folder: str, ctx: Optional[int], batch: int, dtype: str, block_si
     state_bytes = (batch + 1) * state_per_slot      # one row per request and the scratch row of padding entries
     workspace = 2048 * (int(emb["width"]) * 4 + int(emb["vocab"]) * 4) + 256 * 1024 * 1024
     total = weight_bytes + kv_bytes + state_bytes + workspace + DEVICE_RESERVE
-    # a decode step reads every matrix once (the embedding table only when it is also the head)
+    # a decode step reads every matrix once for each run of its layer (the embedding table only when it is also the head)
     step_weights = matrix_bytes * (matrix_elements - (0 if tied else embedding_elements)) // max(matrix_elements, 1)
     linear_elements = matrix_elements - embedding_elements - (0 if tied else head_elements)
     plan = {

@@ -65,6 +65,21 @@ def declare_model(config: ModelConfig) -> List[TensorSpec]:
     return specs
 
 
+def tensor_reads(config: ModelConfig) -> Dict[str, int]:
+    """How often a step reads each tensor that belongs to a layer or to the rejoining part: once for every entry of the run
+    order that uses it."""
+    schedule, layers = config.schedule(), config.layer_specs()
+    reads: Dict[str, int] = {}
+    for index, layer in enumerate(layers):
+        runs = sum(entry.layer == index for entry in schedule)
+        for tensor in part_class("block", layer.block).declare(layer):
+            reads[tensor.name] = runs
+    rejoin = config.rejoin_spec()
+    for tensor in part_class("rejoin", rejoin.kind).declare(rejoin, "") if rejoin is not None else ():
+        reads[tensor.name] = sum(entry.rejoins for entry in schedule)
+    return reads
+
+
 def check_model(config: ModelConfig, dtype) -> None:
     """Raise ``UnsupportedError`` if some part of ``config``'s model has a size that no kernel takes in a run of
     ``dtype``.  Touches no GPU and reads no weight: it is what opening a model does first."""
